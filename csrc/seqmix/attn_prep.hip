@@ -1,0 +1,171 @@
+// Input passes of grouped-query attention behind short convolutions, and the pooled blocks of
+// its key/value pool.
+//
+// conv_rope_norm_store_k: one projection buffer holds q (H heads x D) | k (G x D) | v (G x V) of
+// every row.  Each channel goes through a causal convolution over the sequence's last K
+// projected values (those before the portion come from the slot's saved tail, or are zero before
+// position 0); nrot channel pairs (i, i + nrot) of every q / k head are turned by the angle
+// pos * inv_freq[i]; q and k heads are divided by their root mean square, sqrt(mean x^2 + eps);
+// q also takes a factor per head (`temp`), which stands for a factor on that head's scores.  q
+// goes to its own buffer, k | v to the row of the paged pool that the token owns.  Convolution,
+// angles, rotation and norm are fp32.  One wavefront per (row, head).
+//
+// Pooled blocks: block b of a sequence is the P tokens bP .. bP + P - 1; its key and value are the
+// means of theirs as the pool holds them.  A second pool keeps them in the activation type: the
+// page that holds a block's last token t has ceil(page / P) rows in it, row (t % page) / P is the
+// block's.  A block is formed in the step that brings its last token, from the first pool:
+// pool_blocks_k, after every row of the step is stored.  A portion of one token (decode) needs
+// no second pass: its wavefronts read back the block's other tokens, which earlier steps
+// stored, and add their own; they move the convolution's tail forward as well.
+#include "common.h"
+using namespace sm;
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, int V,
+                       const float* __restrict__ cw, int K, float* tail,
+                       const int* __restrict__ ent, const int* __restrict__ row_ent,
+                       const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
+                       float eps, const int* __restrict__ pos, const int* __restrict__ cache_rows,
+                       T* pool, T* __restrict__ q_out, int ldq, T* __restrict__ blk, int P,
+                       const int* __restrict__ bt, int max_pages, int page, int LDS) {
+  extern __shared__ float smem[];
+  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int hh = blockIdx.y * 4 + wave;                 // q heads, then k heads, then v heads
+  const bool on = hh < H + 2 * G;
+  const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
+  const int hd = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
+  const int n = kind == 2 ? V : D;
+  const int c0 = kind == 0 ? hd * D : kind == 1 ? (H + hd) * D : (H + G) * D + hd * V;
+  const int C = (H + G) * D + G * V, W = G * (D + V);
+  float* s = smem + wave * LDS;
+  const int e = row_ent[r];
+  const Entry en = load_entry(ent, e);
+  const int t = r - en.row0;
+  const bool single = en.n == 1;
+  if (on)
+    for (int i = lane; i < n; i += 64) {
+      const int c = c0 + i;
+      const float* w = cw + (size_t)c * K;
+      float* tl = tail + (size_t)en.slot * (K - 1) * C + c;
+      float acc = 0.0f;
+      for (int kk = 0; kk < K; kk++) {
+        const int q = t - (K - 1) + kk;
+        float v = 0.0f;
+        if (q >= 0) v = ldf(proj, (size_t)(en.row0 + q) * ldp + c);
+        else if (en.start > 0) v = tl[(size_t)(K - 1 + q) * C];
+        acc += w[kk] * v;
+        // the tail after this token is its window without the oldest value (a slot is written
+        // after the value it held has been used)
+        if (single && kk > 0) tl[(size_t)(kk - 1) * C] = v;
+      }
+      s[i] = acc;
+    }
+  __syncthreads();
+  if (!on) return;
+  const int p = pos[r];
+  T* crow = pool + (size_t)cache_rows[r] * W;
+  T* dst = kind == 0 ? q_out + (size_t)r * ldq + hd * D : kind == 1 ? crow + hd * D
+                                                                    : crow + G * D + hd * V;
+  float rs = 1.0f;
+  if (kind < 2) {
+    float ss = 0.0f;
+    for (int j = lane; j < nrot; j += 64) {   // a pair stays with one lane
+      const float a = s[j], b = s[j + nrot];
+      float sn, cs;
+      sincosf((float)p * inv_freq[j], &sn, &cs);
+      const float x = a * cs - b * sn, y = b * cs + a * sn;
+      s[j] = x;
+      s[j + nrot] = y;
+      ss += x * x + y * y;
+    }
+    for (int i = 2 * nrot + lane; i < n; i += 64) ss += s[i] * s[i];
+    ss = wave_sum(ss);
+    rs = 1.0f / sqrtf(ss / (float)n + eps);
+    if (kind == 0 && temp) rs *= temp[hd];
+  }
+  // another lane may have turned the value this lane stores
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  const bool ends = blk && single && kind > 0 && (p + 1) % P == 0;
+  const int wo = kind == 1 ? hd * D : G * D + hd * V;      // place in a pool row
+  const int* pages = bt + (size_t)e * max_pages;
+  T* brow = ends ? blk + ((size_t)pages[p / page] * ((page + P - 1) / P) + (p % page) / P) * W + wo
+                 : nullptr;
+  for (int i = lane; i < n; i += 64) {
+    T own;
+    stf(&own, 0, s[i] * rs);
+    dst[i] = own;
+    if (ends) {
+      float sum = 0.0f;
+      for (int j = p - P + 1; j < p; j++)
+        sum += ldf(pool, ((size_t)pages[j / page] * page + j % page) * W + wo + i);
+      stf(brow, i, (sum + ldf(&own, 0)) / (float)P);
+    }
+  }
+}
+
+// blocks that the step's portions of more than one token complete; one workgroup per (block,
+// entry), grid.x covers the entry with most of them
+template <typename T>
+__global__ void __launch_bounds__(256)
+pool_blocks_k(const T* __restrict__ pool, int W, T* __restrict__ blk, int P,
+              const int* __restrict__ ent, const int* __restrict__ bt, int max_pages, int page) {
+  const int e = blockIdx.y;
+  const Entry en = load_entry(ent, e);
+  const int last = (en.start / P + blockIdx.x) * P + P - 1;
+  if (en.n < 2 || last >= en.start + en.n) return;
+  const int* pages = bt + (size_t)e * max_pages;
+  T* brow = blk + ((size_t)pages[last / page] * ((page + P - 1) / P) + (last % page) / P) * W;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    float sum = 0.0f;
+    int j = last - P + 1;
+    for (; j + 4 <= last + 1; j += 4) {   // four loads in flight, added in order
+      float v[4];
+#pragma unroll
+      for (int u = 0; u < 4; u++)
+        v[u] = ldf(pool, ((size_t)pages[(j + u) / page] * page + (j + u) % page) * W + c);
+#pragma unroll
+      for (int u = 0; u < 4; u++) sum += v[u];
+    }
+    for (; j <= last; j++) sum += ldf(pool, ((size_t)pages[j / page] * page + j % page) * W + c);
+    stf(brow, c, sum / (float)P);
+  }
+}
+
+extern "C" {
+
+int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, int V,
+                                const float* cw, int K, float* tail, const int* ent,
+                                const int* row_ent, const float* inv_freq, int nrot,
+                                const float* temp, float eps, const int* pos,
+                                const int* cache_rows, void* pool, void* q_out, int ldq, void* blk,
+                                int P, const int* bt, int max_pages, int page, int R, int f32,
+                                hipStream_t st) {
+  if (R <= 0) return 0;
+  if (H < 1 || G < 1 || D < 1 || V < 1 || K < 1 || nrot < 0 || 2 * nrot > D || page < 1 ||
+      (blk && P < 1))
+    return (int)hipErrorInvalidValue;
+  const int LDS = D > V ? D : V;
+  if ((size_t)4 * LDS * 4 > 64 * 1024) return (int)hipErrorInvalidValue;
+  dim3 grid(R, (H + 2 * G + 3) / 4);
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL(conv_rope_norm_store_k<T>, grid, dim3(256),
+                                         (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, D, V,
+                                         cw, K, tail, ent, row_ent, inv_freq, nrot, temp, eps, pos,
+                                         cache_rows, (T*)pool, (T*)q_out, ldq, (T*)blk, P, bt,
+                                         max_pages, page, LDS));
+  return (int)hipGetLastError();
+}
+
+// max_blocks: the most blocks a portion of the step completes
+int p2p_sm_pool_blocks(const void* pool, int W, void* blk, int P, const int* ent, int E,
+                       int max_blocks, const int* bt, int max_pages, int page, int f32,
+                       hipStream_t st) {
+  if (E <= 0 || max_blocks <= 0) return 0;
+  if (P < 1 || W < 1 || page < 1) return (int)hipErrorInvalidValue;
+  dim3 grid(max_blocks, E);
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL(pool_blocks_k<T>, grid, dim3(256), 0, st, (const T*)pool,
+                                         W, (T*)blk, P, ent, bt, max_pages, page));
+  return (int)hipGetLastError();
+}
+
+}  // extern "C"

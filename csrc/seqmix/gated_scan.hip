@@ -19,6 +19,10 @@
 // in LDS, and the epilogue sums them per token.  The head's o is RMS-normalised, weighted per
 // channel of the head and gated by a sigmoid.
 //
+// Lightning attention is the plain write with one constant decay per head on q = silu(.),
+// k = silu(.), v = silu(.); its norm spans all heads of a row, so o leaves in fp32 as it is.  This
+// kernel walks its decode steps and short portions; long ones go through lightning.hip.
+//
 // The value columns of S are independent.  A wavefront covers 16 columns x 4 slices of the key
 // index; lane (c, s) keeps rows s*DQ .. s*DQ+DQ-1 of column c in registers (NC columns, 16
 // apart, in the general form of the kernel), and the sums over the key index (S^T k before
@@ -53,6 +57,8 @@ struct ScanArgs {
   // matrix memory: proj = [q (H*D) | k (H*D) | v (H*V) | gate (H*V) | ...] and the
   // coefficients (a_t, b_t, exp(-m_t)) fp32 [rows, H, 3]
   const float* coef;
+  // lightning: proj = [q (H*D) | k (H*D) | v (H*V) | ...], decay fp32 [H]; out is fp32
+  const float* decay;
   int VS;   // value columns of the state: V, or V + 1 with the normaliser
   // common
   const float* normw; float* state; const int* ent; void* out; int ldo;
@@ -68,9 +74,9 @@ struct ScanArgs {
   float* chunk_trans;   // [chunks, H, D, D]
 };
 
-template <typename T, int DQ, int KIND, int NC>   // KIND 0: plain write (HGRN2), 1: delta rule, 2: matrix memory
+template <typename T, int DQ, int KIND, int NC>   // KIND 0: plain write (HGRN2), 1: delta rule, 2: matrix memory, 3: lightning
 __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
-  constexpr bool DELTA = KIND == 1, MEM = KIND == 2;
+  constexpr bool DELTA = KIND == 1, MEM = KIND == 2, LIGHT = KIND == 3;
   constexpr int DKP = 4 * DQ;   // padded key index (zero filled in LDS)
   constexpr int WC = 16 * NC;   // columns per wavefront: a lane keeps NC columns, 16 apart
   const int H = a.H, D = a.D, V = a.V, VS = a.VS, CT = a.CT, mode = a.mode;
@@ -147,6 +153,12 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
           vq = ldf(proj, row * a.ldp + h * D + i) * qscale;
           vk = cf[1] * ldf(proj, row * a.ldp + H * D + h * D + i);
           vg = cf[0];
+        } else if (LIGHT) {
+          float qr = ldf(proj, row * a.ldp + h * D + i);
+          float kr = ldf(proj, row * a.ldp + H * D + h * D + i);
+          vq = qr * sigmoidf_(qr);
+          vk = kr * sigmoidf_(kr);
+          vg = a.decay[h];
         } else {
           float qr = ldf(proj, row * a.ldp + h * D + i);
           vq = qr * sigmoidf_(qr);
@@ -164,6 +176,7 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
         float vv = 0.0f;
         if (i < V) vv = DELTA ? a.conv[row * a.ldc + 2 * a.G * D + h * V + i]
                               : ldf(proj, row * a.ldp + 2 * H * D + h * V + i);
+        if (LIGHT) vv *= sigmoidf_(vv);
         sv[idx] = vv;
       }
     if (DELTA) {
@@ -276,6 +289,11 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
     if (mode == 0 || mode == 2)
     for (int t = wave; t < ct; t += nw) {
       size_t row = (size_t)(en.row0 + t0 + t);
+      if (LIGHT) {
+        for (int i = lane; i < V; i += 64)
+          ((float*)a.out)[row * a.ldo + h * V + i] = so[t * VP + i];
+        continue;
+      }
       float den = 1.0f;
       if (MEM) {
         float nq = 0.0f;
@@ -537,6 +555,17 @@ static int launch_chunked(ScanArgs a, const int* vent, int NV, const int* cent, 
 }
 
 extern "C" {
+
+// portions in one pass; out fp32 [R, H*V] (no norm)
+int p2p_sm_lightning_scan(const void* proj, int ldp, const float* decay, float* state,
+                          const int* ent, int E, float* out, int ldo, int H, int D, int V, int f32,
+                          hipStream_t st) {
+  ScanArgs a = {};
+  a.proj = proj; a.ldp = ldp; a.decay = decay;
+  a.state = state; a.ent = ent; a.out = out; a.ldo = ldo;
+  a.H = H; a.G = H; a.D = D; a.V = V;
+  return launch_scan<3>(a, E, f32, st);
+}
 
 int p2p_sm_hgrn2_scan(const void* proj, int ldp, const float* lower, const float* fb,
                       const float* normw, float* state, const int* ent, int E, void* out, int ldo,

@@ -8,15 +8,18 @@
 //          dt of a chunk of tokens go through LDS.  Long portions run as chunks side by
 //          side (modes 1 and 2 + mamba_combine_k).
 //   tail : rolls the convolution tail forward after the scan.
+// The convolution serves other layers too: it writes fp32 or activation-typed rows.
 #include "common.h"
 using namespace sm;
 
-template <typename T>
+// roll: a portion of one token (decode) also moves its tail forward here, every thread that of
+// its own channel; the tails of longer portions wait for mamba_tail_k (other rows read them).
+template <typename T, typename TO>
 __global__ void mamba_conv_k(const T* __restrict__ zx, int ldz, int xoff,
                              const float* __restrict__ cw, const float* __restrict__ cb,
-                             const float* __restrict__ tail, const int* __restrict__ ent,
-                             const int* __restrict__ row_ent, float* __restrict__ out, int R,
-                             int C, int K) {
+                             float* tail, const int* __restrict__ ent,
+                             const int* __restrict__ row_ent, TO* __restrict__ out, int ldo,
+                             int C, int K, int roll) {
   int c = blockIdx.x * blockDim.x + threadIdx.x;
   int r = blockIdx.y;
   if (c >= C) return;
@@ -30,7 +33,13 @@ __global__ void mamba_conv_k(const T* __restrict__ zx, int ldz, int xoff,
     else if (en.start > 0) val = tail[((size_t)en.slot * (K - 1) + (K - 1 + q)) * C + c];
     acc += cw[(size_t)c * K + kk] * val;
   }
-  out[(size_t)r * C + c] = acc * sigmoidf_(acc);
+  stf(out, (size_t)r * ldo + c, acc * sigmoidf_(acc));
+  if (roll && en.n == 1) {
+    float* tl = tail + (size_t)en.slot * (K - 1) * C + c;
+    for (int j = 0; j < K - 1; j++)
+      tl[(size_t)j * C] = j + 1 < K - 1 ? (en.start > 0 ? tl[(size_t)(j + 1) * C] : 0.0f)
+                                        : ldf(zx, (size_t)r * ldz + xoff + c);
+  }
 }
 
 // One thread owns NSUB consecutive state rows of one value column: thread (p, ns) holds
@@ -164,11 +173,11 @@ __global__ void mamba_combine_k(float* __restrict__ tmp, const float* __restrict
 // a slot it has already written
 template <typename T>
 __global__ void mamba_tail_k(const T* __restrict__ zx, int ldz, int xoff, float* __restrict__ tail,
-                             const int* __restrict__ ent, int C, int K) {
+                             const int* __restrict__ ent, int C, int K, int skip_single) {
   int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= C) return;
   Entry en = load_entry(ent, blockIdx.y);
-  if (en.n <= 0) return;
+  if (en.n <= 0 || (skip_single && en.n == 1)) return;
   float* tl = tail + (size_t)en.slot * (K - 1) * C;
   for (int j = 0; j < K - 1; j++) {
     int q = en.n + j - (K - 1);
@@ -200,12 +209,19 @@ static int launch_ms(const float* conv, int C, const void* zx, int ldz, int xoff
 extern "C" {
 
 int p2p_sm_mamba_conv(const void* zx, int ldz, int xoff, const float* cw, const float* cb,
-                      const float* tail, const int* ent, const int* row_ent, float* out, int R,
-                      int C, int K, int f32, hipStream_t st) {
+                      float* tail, const int* ent, const int* row_ent, void* out, int ldo,
+                      int out_f32, int R, int C, int K, int roll, int f32, hipStream_t st) {
   if (R <= 0) return 0;
+  if (K < 1) return (int)hipErrorInvalidValue;
   dim3 g((C + 255) / 256, R), b(256);
-  SM_DISPATCH_T(f32, hipLaunchKernelGGL(mamba_conv_k<T>, g, b, 0, st, (const T*)zx, ldz, xoff, cw,
-                                         cb, tail, ent, row_ent, out, R, C, K));
+  if (out_f32)
+    SM_DISPATCH_T(f32, hipLaunchKernelGGL((mamba_conv_k<T, float>), g, b, 0, st, (const T*)zx, ldz,
+                                           xoff, cw, cb, tail, ent, row_ent, (float*)out, ldo, C,
+                                           K, roll));
+  else
+    SM_DISPATCH_T(f32, hipLaunchKernelGGL((mamba_conv_k<T, T>), g, b, 0, st, (const T*)zx, ldz,
+                                           xoff, cw, cb, tail, ent, row_ent, (T*)out, ldo, C, K,
+                                           roll));
   return (int)hipGetLastError();
 }
 
@@ -232,7 +248,8 @@ int p2p_sm_mamba_scan_mode(const float* conv, int C, const void* zx, int ldz, in
 int p2p_sm_mamba_scan(const float* conv, int C, const void* zx, int ldz, int xoff, int dtoff,
                       const float* dt_bias, const float* A_log, const float* Dp, float* state,
                       float* tail, const int* ent, int E, float* y, int H, int P, int N, int G,
-                      int K, int f32, hipStream_t st) {  return p2p_sm_mamba_scan_mode(conv, C, zx, ldz, xoff, dtoff, dt_bias, A_log, Dp, state, tail,
+                      int K, int f32, hipStream_t st) {
+  return p2p_sm_mamba_scan_mode(conv, C, zx, ldz, xoff, dtoff, dt_bias, A_log, Dp, state, tail,
                                 ent, E, y, H, P, N, G, K, 0, nullptr, f32, st);
 }
 
@@ -258,11 +275,11 @@ int p2p_sm_mamba_scan_chunked(const float* conv, int C, const void* zx, int ldz,
 }
 
 int p2p_sm_mamba_tail(const void* zx, int ldz, int xoff, float* tail, const int* ent, int E, int C,
-                      int K, int f32, hipStream_t st) {
+                      int K, int skip_single, int f32, hipStream_t st) {
   if (E <= 0 || K <= 1) return 0;
   dim3 g((C + 255) / 256, E), b(256);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(mamba_tail_k<T>, g, b, 0, st, (const T*)zx, ldz, xoff, tail,
-                                        ent, C, K));
+                                        ent, C, K, skip_single));
   return (int)hipGetLastError();
 }
 

@@ -70,8 +70,8 @@ __global__ void rmsnorm_k(const TI* __restrict__ x, int ldx, const float* __rest
   }
 }
 
-// x += y / sqrt(mean(y^2) + eps) * w * ls   (x fp32 residual); with w2 also the next
-// sublayer's input h = x / sqrt(mean(x^2) + eps) * w2 from the updated row
+// x += y / sqrt(mean(y^2) + eps) * w * ls   (x fp32 residual); with h also the next sublayer's
+// input from the updated row: x / sqrt(mean(x^2) + eps) * w2, or without w2 the row as it is
 template <typename T>
 __global__ void norm_scale_add_k(float* __restrict__ x, const T* __restrict__ y, int ldy,
                                  const float* __restrict__ w, const float* __restrict__ ls,
@@ -104,7 +104,16 @@ __global__ void norm_scale_add_k(float* __restrict__ x, const T* __restrict__ y,
       if (i < n) xr[i] = xv[k];
       s2 += xv[k] * xv[k];
     }
-    if (!w2) return;
+    if (!w2) {
+      if (h) {
+#pragma unroll
+        for (int k = 0; k < NV; k++) {
+          int i = threadIdx.x + k * blockDim.x;
+          if (i < n) stf(h, (size_t)r * ldh + i, xv[k]);
+        }
+      }
+      return;
+    }
     s2 = block_sum(s2, red);
     float r2 = 1.0f / sqrtf(s2 / (float)n + eps);
 #pragma unroll
@@ -125,6 +134,7 @@ __global__ void norm_scale_add_k(float* __restrict__ x, const T* __restrict__ y,
   for (int i = threadIdx.x; i < n; i += blockDim.x) {
     float v = xr[i] + ldf(yr, i) * rs * (ls ? w[i] * ls[i] : w[i]);
     xr[i] = v;
+    if (h && !w2) stf(h, (size_t)r * ldh + i, v);
     s2 += v * v;
   }
   if (!w2) return;
@@ -385,7 +395,58 @@ __global__ void gate_norm_add_k(float* __restrict__ x, const T* __restrict__ y, 
   }
 }
 
+// out = x / sqrt(mean(x^2) + eps) * w * sigmoid(g): the norm of a whole fp32 row (all heads of a
+// recurrence together) with a gate per channel, on the way into an output projection
+template <typename T>
+__global__ void norm_gate_k(const float* __restrict__ x, int ldx, const float* __restrict__ w,
+                            const T* __restrict__ g, int ldg, T* __restrict__ out, int ldo, int n,
+                            float eps) {
+  __shared__ float red[16];
+  const int r = blockIdx.x;
+  const float* xr = x + (size_t)r * ldx;
+  const T* gr = g + (size_t)r * ldg;
+  T* o = out + (size_t)r * ldo;
+  if (n <= NV * (int)blockDim.x) {
+    float v[NV], m[NV];
+    float ss = 0.0f;
+#pragma unroll
+    for (int k = 0; k < NV; k++) {
+      int i = threadIdx.x + k * blockDim.x;
+      int ic = i < n ? i : 0;
+      v[k] = xr[ic];
+      m[k] = w[ic] * sigmoidf_(ldf(gr, ic));
+    }
+#pragma unroll
+    for (int k = 0; k < NV; k++) {
+      if (threadIdx.x + k * blockDim.x >= (unsigned)n) v[k] = 0.0f;
+      ss += v[k] * v[k];
+    }
+    ss = block_sum(ss, red);
+    float rs = 1.0f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+    for (int k = 0; k < NV; k++) {
+      int i = threadIdx.x + k * blockDim.x;
+      if (i < n) stf(o, i, v[k] * rs * m[k]);
+    }
+    return;
+  }
+  float ss = 0.0f;
+  for (int i = threadIdx.x; i < n; i += blockDim.x) ss += xr[i] * xr[i];
+  ss = block_sum(ss, red);
+  float rs = 1.0f / sqrtf(ss / (float)n + eps);
+  for (int i = threadIdx.x; i < n; i += blockDim.x)
+    stf(o, i, xr[i] * rs * w[i] * sigmoidf_(ldf(gr, i)));
+}
+
 extern "C" {
+
+int p2p_sm_norm_gate(const float* x, int ldx, const float* w, const void* g, int ldg, void* out,
+                     int ldo, int R, int n, float eps, int f32, hipStream_t st) {
+  if (R <= 0 || n <= 0) return 0;
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL(norm_gate_k<T>, dim3(R), dim3(256), 0, st, x, ldx, w,
+                                         (const T*)g, ldg, (T*)out, ldo, n, eps));
+  return (int)hipGetLastError();
+}
 
 int p2p_sm_embed_rows(const void* embed, const int* ids, float* out, void* h, int ldh, int R,
                       int W, float scale, int f32, hipStream_t st) {

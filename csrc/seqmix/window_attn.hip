@@ -17,9 +17,13 @@
 // maximum starts at sink_h and the running sum at 1 (without a sink: an ordinary softmax).
 // Optional steps on a score s of query position i and key position j, in this order:
 // cap * tanh(s / cap) (cap > 0), and s - r1_h * ln(1 + r2_h * (i - j)) (r1, r2 given).  Optional
-// head gate: head h of row r leaves multiplied by sigmoid(gate[r, h]).  One block per (query
-// row, key/value head): the heads of the group share the key and value tiles, which stream
-// through LDS with an online softmax.
+// gate: head h of row r leaves multiplied by sigmoid(gate[r, h]), or (gate_pc) its channel c by
+// sigmoid(gate[r, h * V + c]).  Optional pooled blocks (`blk`): beside the tokens of the window a
+// row sees one key and value for every block of P tokens that lies wholly before the window,
+// (i - win + 1) / P of them, stored in a pool of their own (the row of the block with last token
+// t: the page that holds t times ceil(page / P), plus (t % page) / P); blocks and tokens share
+// the softmax.  One block per (query row, key/value head): the heads of the group share the
+// key and value tiles, which stream through LDS with an online softmax.
 //
 // rope_rows_k: turns the channel pairs (2i, 2i+1) of a stretch of every head by pos * inv_freq[i]
 // and writes them to another place (its own rows or scattered ones).  qtemp_kv_store_k: the
@@ -202,7 +206,8 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
               const int* __restrict__ pos, const float* __restrict__ sink, float scale, int win,
               T* __restrict__ out, int ldo, int H, int G, int D, int V, int page, int TK,
               float out_scale, int HB, float cap, const float* __restrict__ r1,
-              const float* __restrict__ r2, const T* __restrict__ gate, int ldg) {
+              const float* __restrict__ r2, const T* __restrict__ gate, int ldg, int gate_pc,
+              const T* __restrict__ blk, int P) {
   extern __shared__ float smem[];
   // a block takes up to HB query heads of one key/value head (all of them when they fit)
   const int nhb = (H / G + HB - 1) / HB;
@@ -219,7 +224,19 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
   const int r = blockIdx.x, tid = threadIdx.x;
   const int p = pos[r];
   const int* pages = bt + (size_t)row_ent[r] * max_pages;
-  const int j_lo = max(0, p - win + 1);
+  const int w_lo = max(0, p - win + 1);
+  // keys are walked as pooled blocks 0 .. nb-1 followed by tokens w_lo .. p: place u of that list
+  // is token u + w_lo - nb from place nb on
+  const int nb = blk ? w_lo / P : 0, shift = w_lo - nb, SB = blk ? (page + P - 1) / P : 1;
+  const int last = p - shift;
+  auto key_row = [&](int u) {
+    if (u < nb) {
+      const int t = u * P + P - 1;
+      return blk + ((size_t)pages[t / page] * SB + (t % page) / P) * ldpool;
+    }
+    const int j = u + shift;
+    return pool + ((size_t)pages[j / page] * page + (j % page)) * ldpool;
+  };
   for (int idx = tid; idx < HG * D; idx += WA_THREADS)
     sq[idx] = ldf(q, (size_t)r * ldq + (size_t)h0 * D + idx);
   if (tid < HG) {
@@ -230,20 +247,16 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
 #pragma unroll
   for (int a = 0; a < WA_ACC; a++) acc[a] = 0.0f;
   const int npair = HG * V;
-  for (int j0 = j_lo; j0 <= p; j0 += TK) {
-    int nk = min(TK, p + 1 - j0);
+  for (int j0 = 0; j0 <= last; j0 += TK) {
+    int nk = min(TK, last + 1 - j0);
     __syncthreads();  // previous tile fully consumed (and sq / sm_ / sl initialised)
     for (int idx = tid; idx < nk * D; idx += WA_THREADS) {
       int jj = idx / D, c = idx % D;
-      int j = j0 + jj;
-      size_t tok = (size_t)pages[j / page] * page + (j % page);
-      sk[jj * ldk + c] = ldf(pool, tok * ldpool + (size_t)g * D + c);
+      sk[jj * ldk + c] = ldf(key_row(j0 + jj), (size_t)g * D + c);
     }
     for (int idx = tid; idx < nk * V; idx += WA_THREADS) {
       int jj = idx / V, c = idx % V;
-      int j = j0 + jj;
-      size_t tok = (size_t)pages[j / page] * page + (j % page);
-      sv[jj * ldv + c] = ldf(pool, tok * ldpool + (size_t)G * D + (size_t)g * V + c);
+      sv[jj * ldv + c] = ldf(key_row(j0 + jj), (size_t)G * D + (size_t)g * V + c);
     }
     __syncthreads();
     for (int idx = tid; idx < HG * TK; idx += WA_THREADS) {
@@ -256,7 +269,7 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
         for (int i = 0; i < D; i++) d += qh[i] * kr[i];
         s = d * scale;
         if (cap > 0.0f) s = cap * tanhf(s / cap);
-        if (r1) s -= r1[h0 + h] * log1pf(r2[h0 + h] * (float)(p - (j0 + jj)));
+        if (r1) s -= r1[h0 + h] * log1pf(r2[h0 + h] * (float)(last - (j0 + jj)));
       }
       sp[idx] = s;
     }
@@ -298,7 +311,8 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
     if (idx < npair) {
       int h = idx / V;
       float o = acc[a] / sl[h] * out_scale;
-      if (gate) o *= sigmoidf_(ldf(gate, (size_t)r * ldg + h0 + h));
+      if (gate)
+        o *= sigmoidf_(ldf(gate, (size_t)r * ldg + (gate_pc ? (size_t)h0 * V + idx : h0 + h)));
       stf(out, (size_t)r * ldo + (size_t)h0 * V + idx, o);
     }
   }
@@ -358,9 +372,11 @@ int p2p_sm_window_attn(const void* q, int ldq, const void* pool, const int* bt, 
                        const int* row_ent, const int* pos, const float* sink, float scale, int win,
                        void* out, int ldo, int R, int H, int G, int D, int V, int page,
                        float out_scale, float cap, const float* r1, const float* r2,
-                       const void* gate, int ldg, int f32, hipStream_t st) {
+                       const void* gate, int ldg, int gate_pc, const void* blk, int P, int f32,
+                       hipStream_t st) {
   if (R <= 0) return 0;
-  if (H < 1 || G < 1 || H % G || D < 1 || V < 1 || win < 1 || (r1 && !r2) || cap < 0.0f)
+  if (H < 1 || G < 1 || H % G || D < 1 || V < 1 || win < 1 || (r1 && !r2) || cap < 0.0f ||
+      (blk && (P < 1 || r1)))   // a distance penalty needs positions, which blocks do not have
     return (int)hipErrorInvalidValue;
   int HG = H / G, TK = WA_TK, HB = HG;
   auto lds = [&](int tk, int hb) {
@@ -378,7 +394,8 @@ int p2p_sm_window_attn(const void* q, int ldq, const void* pool, const int* bt, 
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(window_attn_k<T>, grid, dim3(WA_THREADS), lds(TK, HB), st,
                                          (const T*)q, ldq, (const T*)pool, bt, max_pages, row_ent,
                                          pos, sink, scale, win, (T*)out, ldo, H, G, D, V, page, TK,
-                                         out_scale, HB, cap, r1, r2, (const T*)gate, ldg));
+                                         out_scale, HB, cap, r1, r2, (const T*)gate, ldg, gate_pc,
+                                         (const T*)blk, P));
   return (int)hipGetLastError();
 }
 

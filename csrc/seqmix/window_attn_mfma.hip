@@ -2,8 +2,12 @@
 // sums).  Same inputs and outputs as window_attn_k: pool row = [k of G heads | v of G heads],
 // query head h reads key/value head h / (H/G), causal sliding window of `win` keys, softmax
 // denominator with one more term exp(sink_h); optionally scores capped by cap * tanh(s / cap),
-// a per-head penalty r1_h * ln(1 + r2_h * distance) taken off them, and every head's result
-// multiplied by sigmoid(gate[row, head]).
+// a per-head penalty r1_h * ln(1 + r2_h * distance) taken off them, every head's result
+// multiplied by sigmoid(gate[row, head]) or channel by channel by sigmoid(gate[row, head * V + c]),
+// and one more key and value per block of P tokens that lies wholly before a row's window (BLK
+// instances; see window_attn_k for where they are stored).  The keys of a row group are then its
+// blocks followed by its tokens, one list that is cut into tiles (and runs) without regard to
+// where the one ends and the other begins.
 //
 // The query heads of one key/value head attend to the same keys, so (row, head) pairs are the M
 // dimension: one wavefront owns 16 pairs -- RW consecutive rows of one sequence portion x HS
@@ -32,7 +36,7 @@ __device__ __forceinline__ float fast_tanh(float x) {
 
 #define WM_LDK 36   // keys per transposed value row in LDS (32 + padding), in bf16
 
-template <int NK, int NV2>  // D padded to NK * 32, V padded to NV2 * 32
+template <int NK, int NV2, bool BLK>  // D padded to NK * 32, V padded to NV2 * 32
 __global__ void __launch_bounds__(64)
 window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__ pool,
                    const int* __restrict__ bt, int max_pages, const int* __restrict__ row_ent,
@@ -41,7 +45,8 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
                    int ldo, int H, int G, int D, int V, int page, int HS, int splits,
                    float* __restrict__ part, float out_scale, float cap,
                    const float* __restrict__ r1, const float* __restrict__ r2,
-                   const bf16* __restrict__ gate, int ldg) {
+                   const bf16* __restrict__ gate, int ldg, int gate_pc,
+                   const bf16* __restrict__ blk, int P) {
   constexpr int DP = NK * 32;        // padded key size
   constexpr int VP = NV2 * 32;       // padded value size
   constexpr int NT = NV2 * 2;        // 16-wide output column tiles
@@ -54,8 +59,7 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
   const int HG = H / G, hblocks = (HG + HS - 1) / HS;
   const int g = blockIdx.y / hblocks, hb0 = (blockIdx.y % hblocks) * HS;   // head slots hb0 ..
   const int ldpool = G * (D + V);
-  const bf16* kbase = pool + (size_t)g * D;
-  const bf16* vbase = pool + (size_t)G * D + (size_t)g * V;
+  const size_t koff = (size_t)g * D, voff = (size_t)G * D + (size_t)g * V;
   // this lane's pair (as a column of S^T and a row of P)
   const int prow = n16 / HS, phs = hb0 + n16 % HS;
   const bool pvalid = prow < nr && phs < HG;
@@ -63,6 +67,17 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
   const int ppos = pvalid ? pos[r0 + prow] : -1;
   const int* pages = bt + (size_t)row_ent[r0] * max_pages;
   int j_lo = max(0, pos[r0] - win + 1), j_hi = pos[r0 + nr - 1];
+  // BLK: places 0 .. nb-1 are blocks (all that the group's last row sees), place u >= nb is token
+  // u + shift; otherwise places are token positions
+  int nb = 0, shift = 0, pnb = 0, SB = 1;
+  if constexpr (BLK) {
+    nb = max(0, j_hi - win + 1) / P;
+    pnb = pvalid ? max(0, ppos - win + 1) / P : 0;   // blocks this lane's row sees
+    SB = (page + P - 1) / P;
+    shift = j_lo - nb;
+    j_lo = 0;
+    j_hi -= shift;
+  }
   if (splits > 1) {
     // this block takes one run of 32-key tiles of the window; partial results go to `part`
     int tiles = (j_hi - j_lo) / 32 + 1;
@@ -98,19 +113,27 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
 #pragma unroll
     for (int sub = 0; sub < 2; sub++) {
       int j = j0 + sub * 16 + n16;   // the key this lane loads
-      size_t tok = 0;
       bool have = j <= j_hi;
-      if (have) tok = ((size_t)pages[j / page] * page + (j % page)) * ldpool;
+      const bf16* row = pool;
+      if (have) {
+        if (BLK && j < nb) {
+          const int t = j * P + P - 1;
+          row = blk + ((size_t)pages[t / page] * SB + (t % page) / P) * ldpool;
+        } else {
+          const int jt = j + shift;
+          row = pool + ((size_t)pages[jt / page] * page + (jt % page)) * ldpool;
+        }
+      }
       uint4 kf[NK], vf[NV2];
 #pragma unroll
       for (int kk = 0; kk < NK; kk++) {
         int c8 = kk * 32 + quad * 8;
-        kf[kk] = (have && c8 < D) ? *(const uint4*)(kbase + tok + c8) : make_uint4(0, 0, 0, 0);
+        kf[kk] = (have && c8 < D) ? *(const uint4*)(row + koff + c8) : make_uint4(0, 0, 0, 0);
       }
 #pragma unroll
       for (int kk = 0; kk < NV2; kk++) {
         int c8 = kk * 32 + quad * 8;
-        vf[kk] = (have && c8 < V) ? *(const uint4*)(vbase + tok + c8) : make_uint4(0, 0, 0, 0);
+        vf[kk] = (have && c8 < V) ? *(const uint4*)(row + voff + c8) : make_uint4(0, 0, 0, 0);
       }
       f32x4 sa = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -142,7 +165,13 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
 #pragma unroll
       for (int i = 0; i < 4; i++) {
         int j = j0 + sub * 16 + quad * 4 + i;
-        bool ok = pvalid && j <= ppos && j > ppos - win && j <= j_hi;
+        bool ok;
+        if (BLK) {
+          const int jt = j + shift;
+          ok = pvalid && j <= j_hi && (j < nb ? j < pnb : jt <= ppos && jt > ppos - win);
+        } else {
+          ok = pvalid && j <= ppos && j > ppos - win && j <= j_hi;
+        }
         float v = -INFINITY;
         if (ok) {
           v = s[sub][i] * scale;
@@ -218,11 +247,16 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
     if (mr < nr && ms < HG) {
       bf16* o = out + (size_t)(r0 + mr) * ldo + (size_t)(g * HG + ms) * V;
       float gv = inv[i];
-      if (gate) gv *= sigmoidf_(__bfloat162float(gate[(size_t)(r0 + mr) * ldg + g * HG + ms]));
+      const bf16* gr = gate + (size_t)(r0 + mr) * ldg + (size_t)(g * HG + ms) * (gate_pc ? V : 1);
+      if (gate && !gate_pc) gv *= sigmoidf_(__bfloat162float(*gr));
 #pragma unroll
       for (int t = 0; t < NT; t++) {
         int c = t * 16 + n16;
-        if (c < V) o[c] = __float2bfloat16(acc[t][i] * gv);
+        if (c < V) {
+          float v = acc[t][i] * gv;
+          if (gate && gate_pc) v *= sigmoidf_(__bfloat162float(gr[c]));
+          o[c] = __float2bfloat16(v);
+        }
       }
     }
   }
@@ -233,7 +267,7 @@ window_attn_mfma_k(const bf16* __restrict__ q, int ldq, const bf16* __restrict__
 __global__ void window_attn_merge_k(const float* __restrict__ part, const int* __restrict__ units,
                                     bf16* __restrict__ out, int ldo, int H, int G, int V, int HS,
                                     int splits, int VP, float out_scale,
-                                    const bf16* __restrict__ gate, int ldg) {
+                                    const bf16* __restrict__ gate, int ldg, int gate_pc) {
   __shared__ float sw[65];
   const int r0 = units[2 * blockIdx.x], nr = units[2 * blockIdx.x + 1];
   const int HG = H / G, hblocks = (HG + HS - 1) / HS;
@@ -255,17 +289,21 @@ __global__ void window_attn_merge_k(const float* __restrict__ part, const int* _
     d = wave_sum(d);
     sw[z] = w;
     if (z == 0) {
-      float gv = gate ? sigmoidf_(__bfloat162float(gate[(size_t)(r0 + mr) * ldg + g * HG + ms])) : 1.0f;
+      float gv = gate && !gate_pc
+                     ? sigmoidf_(__bfloat162float(gate[(size_t)(r0 + mr) * ldg + g * HG + ms]))
+                     : 1.0f;
       sw[64] = d > 0.0f ? out_scale * gv / d : 0.0f;
     }
   }
   __syncthreads();
   float inv = sw[64];
   bf16* o = out + (size_t)(r0 + mr) * ldo + (size_t)(g * HG + ms) * V;
+  const bf16* gr = gate && gate_pc ? gate + (size_t)(r0 + mr) * ldg + (size_t)(g * HG + ms) * V : nullptr;
   for (int c = threadIdx.x; c < V; c += blockDim.x) {
+    const float gv = gr ? inv * sigmoidf_(__bfloat162float(gr[c])) : inv;
     float num = 0.0f;
     for (int z = 0; z < splits; z++) num += sw[z] * rec[z * zs + c];
-    o[c] = __float2bfloat16(num * inv);
+    o[c] = __float2bfloat16(num * gv);
   }
 }
 
@@ -294,26 +332,30 @@ int p2p_sm_window_attn_mfma(const void* q, int ldq, const void* pool, const int*
                             int U, const float* sink, float scale, int win, void* out, int ldo,
                             int H, int G, int D, int V, int page, int splits, float* part,
                             float out_scale, float cap, const float* r1, const float* r2,
-                            const void* gate, int ldg, hipStream_t st) {
+                            const void* gate, int ldg, int gate_pc, const void* blk, int P,
+                            hipStream_t st) {
   if (U <= 0) return 0;
   if (H < 1 || G < 1 || H % G || D < 8 || D > 256 || D % 8 || V < 8 || V > 256 || V % 8 ||
-      win < 1 || ldq % 8 || (r1 && !r2) || cap < 0.0f)
+      win < 1 || ldq % 8 || (r1 && !r2) || cap < 0.0f || (blk && (P < 1 || r1)))
     return (int)hipErrorInvalidValue;
   if (splits < 1 || splits > 64 || (splits > 1 && !part)) return (int)hipErrorInvalidValue;
   int HG = H / G, HS = head_slots(HG);
   dim3 grid(U, G * ((HG + HS - 1) / HS), splits), block(64);
   int nk = pad32(D), nv = pad32(V);
+#define WMB(NKK, NVV, BLK)                                                                     \
+  hipLaunchKernelGGL((window_attn_mfma_k<NKK, NVV, BLK>), grid, block, shm, st, (const bf16*)q, \
+                     ldq, (const bf16*)pool, bt, max_pages, row_ent, pos, units, sink, scale,  \
+                     win, (bf16*)out, ldo, H, G, D, V, page, HS, splits, part, out_scale, cap, \
+                     r1, r2, (const bf16*)gate, ldg, gate_pc, (const bf16*)blk, P)
 #define WM(NKK, NVV)                                                                           \
   do {                                                                                         \
     size_t shm = (size_t)(16 * (NKK * 32 + 8) + NVV * 32 * WM_LDK) * 2;                        \
-    hipLaunchKernelGGL((window_attn_mfma_k<NKK, NVV>), grid, block, shm, st, (const bf16*)q,   \
-                       ldq, (const bf16*)pool, bt, max_pages, row_ent, pos, units, sink,       \
-                       scale, win, (bf16*)out, ldo, H, G, D, V, page, HS, splits, part,        \
-                       out_scale, cap, r1, r2, (const bf16*)gate, ldg);                        \
+    if (blk) WMB(NKK, NVV, true);                                                              \
+    else WMB(NKK, NVV, false);                                                                 \
     if (splits > 1)                                                                            \
       hipLaunchKernelGGL(window_attn_merge_k, dim3(grid.x, grid.y, 16), dim3(128), 0, st,      \
                          part, units, (bf16*)out, ldo, H, G, V, HS, splits, NVV * 32,          \
-                         out_scale, (const bf16*)gate, ldg);                                   \
+                         out_scale, (const bf16*)gate, ldg, gate_pc);                          \
   } while (0)
 #define WMV(NKK)                 \
   do {                           \
@@ -328,6 +370,7 @@ int p2p_sm_window_attn_mfma(const void* q, int ldq, const void* pool, const int*
   else WMV(8);
 #undef WMV
 #undef WM
+#undef WMB
   return (int)hipGetLastError();
 }
 

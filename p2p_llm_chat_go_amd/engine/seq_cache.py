@@ -6,6 +6,10 @@ list):
   * ``("paged", width)``  -- one vector of ``width`` numbers per token, stored in pages of
     ``PAGE`` tokens drawn from the shared ``PageAllocator`` (page 0 is the null page); a
     sequence's token t lives at ``pages[t // PAGE] * PAGE + t % PAGE`` in every paged layer;
+  * ``("pooled", (width, every))`` -- one vector per block of ``every`` consecutive tokens, beside
+    the layer's paged pool and on the same pages: the page that holds a block's last token t
+    (``t = every - 1, 2 * every - 1, ..``) has ``ceil(PAGE / every)`` rows, row ``t % PAGE // every`` is
+    the block's; a block is written in the step that brings its last token;
   * ``("state", {name: shape})`` -- fp32 tensors per sequence slot, overwritten in place by
     the layer's kernels; a portion that starts at position 0 ignores what the slot held.
 A sequence holds one state slot and a growing list of pages; both return to the free lists
@@ -17,6 +21,7 @@ from __future__ import annotations
 import torch
 
 from ..ops import PAGE
+from ..ops.seqmix import blocks_per_page
 from .kv_cache import PageAllocator, pages_for
 
 
@@ -28,6 +33,17 @@ def layer_specs(specs: list):
             continue
         for kind, what in (spec if isinstance(spec, list) else [spec]):
             yield i, kind, what
+
+
+def numbers_per_page(specs: list) -> int:
+    """Cached numbers a page of tokens takes over all layers."""
+    n = 0
+    for _i, kind, what in layer_specs(specs):
+        if kind == "paged":
+            n += int(what) * PAGE
+        elif kind == "pooled":
+            n += int(what[0]) * blocks_per_page(PAGE, int(what[1]))
+    return n
 
 
 class SlotAllocator:
@@ -66,13 +82,19 @@ class SequenceCache:
         self.num_pages, self.num_slots = num_pages, num_slots
         self.allocator = PageAllocator(num_pages)
         self.slots = SlotAllocator(num_slots)
-        self.paged, self.state = {}, {}
+        self.paged, self.pooled, self.state = {}, {}, {}
         for i, kind, what in layer_specs(specs):
             if kind == "paged":
                 if i in self.paged:
                     raise ValueError("layer %d declares two paged pools" % i)
                 self.paged[i] = torch.zeros(num_pages * PAGE, int(what), device=self.device,
                                             dtype=dtype)
+            elif kind == "pooled":
+                if i in self.pooled:
+                    raise ValueError("layer %d declares two pools of blocks" % i)
+                width, every = int(what[0]), int(what[1])
+                self.pooled[i] = torch.zeros(num_pages * blocks_per_page(PAGE, every), width,
+                                             device=self.device, dtype=dtype)
             elif kind == "state":
                 # one slot more than the allocator hands out: the null slot, where padding rows
                 # of a bucketed (graph-captured) step keep their state, like the null page
@@ -117,7 +139,8 @@ class SequenceCache:
         self.slots.free(seq.slot)
 
     def bytes_per_page(self) -> int:
-        return sum(t.shape[1] * t.element_size() * PAGE for t in self.paged.values())
+        return sum(t.numel() * t.element_size() // self.num_pages
+                   for d in (self.paged, self.pooled) for t in d.values())
 
     def bytes_per_slot(self) -> int:
         return sum(t[0].numel() * 4 for d in self.state.values() for t in d.values())

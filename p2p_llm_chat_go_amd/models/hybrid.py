@@ -14,6 +14,8 @@ is wrapped around the residual stream,
                                                              one weight for all channels; a
                                                              stretch of layers may run several
                                                              passes (``loop``)
+    "post"        x <- x + norm(f(x))                        the sublayers read x itself, a
+                                                             norm on what they produce only
 
 and whether learned absolute positions are added to the token embedding.  Mixers:
 
@@ -43,6 +45,14 @@ and whether learned absolute positions are added to the token embedding.  Mixers
   ``rope_latent_attention``  latent attention with low-rank queries and one rotated key part
                         that the heads share, cached beside the latent; plain causal softmax, one
                         sigmoid gate per head;
+  ``conv_attention``    grouped-query attention behind short convolutions on q, k, v: biased
+                        projections, half-split rotation, unit-RMS query / key heads, a score factor
+                        per head, a sliding window plus one pooled key / value per block of tokens
+                        before it, a gate per channel;
+  ``mamba1``            the first Mamba: short convolution + selective scan with a step size per
+                        channel and N states per channel;
+  ``lightning``         linear attention with one constant decay per head, silu on q, k, v, one
+                        norm over all heads and a sigmoid gate;
   ``parallel``          two mixers side by side on the same input, summed with fixed scales.
 
 Feed-forwards: ``dense`` (silu-gated, or the clamped gated unit when the config gives a
@@ -59,7 +69,9 @@ form (norm weights stored around zero), with gelu-gated dense feed-forwards and 
 squared-relu experts behind a softmax router.  "Tarunex" stacks ``biased_attention`` and
 ``rope_latent_attention`` layers (its config calls them "attention" and "latent_attention") in
 the two-norm parallel form with ``moe_top`` feed-forwards, repeats a stretch of layers, scales
-its embedding and scales and caps its logits.  A checkpoint is a ``config.json`` whose
+its embedding and scales and caps its logits.  "Rasepel" stacks ``mamba1``, ``conv_attention``
+(its config's "attention") and ``lightning`` layers in the post-norm form with clamped dense
+feed-forwards, scales its embedding and reads its logits off the embedding table.  A checkpoint is a ``config.json`` whose
 ``architecture`` names the design and one safetensors file (``load_dir``).
 
 One ``forward`` serves every step: a flat list of token rows cut into entries (portions of
@@ -93,12 +105,14 @@ class LayerSpec:
 
 @dataclasses.dataclass(frozen=True)
 class Design:
-    block: str                # how sublayers sit on the residual stream: "sandwich" | "gated_post" | "parallel"
+    block: str                # how sublayers sit on the residual stream: "sandwich" | "gated_post" |
+                              # "parallel" | "parallel2" | "post"
     positions: str | None     # "learned": a position table is added to the embedding
     norm_offset: float = 0.0  # block and final norm weights are stored minus this (1: around zero)
     ff: tuple = ()            # (config kind, FEEDFORWARDS key) where the two differ
     mixers: tuple = ()        # (config type, MIXERS key) where the two differ
     scalar_norms: bool = False  # block and final norms have one weight for all channels
+    tied_head: bool = False   # the logits are read off the embedding table
 
     def ff_key(self, kind: str) -> str:
         return dict(self.ff).get(kind, kind)
@@ -112,7 +126,9 @@ DESIGNS = {"Regesun": Design("sandwich", "learned"), "Rotutar": Design("gated_po
                              ff=(("dense", "dense_gelu"), ("moe", "moe_softmax"))),
            "Tarunex": Design("parallel2", None, scalar_norms=True, ff=(("moe", "moe_top"),),
                              mixers=(("latent_attention", "rope_latent_attention"),
-                                     ("attention", "biased_attention")))}
+                                     ("attention", "biased_attention"))),
+           "Rasepel": Design("post", None, norm_offset=1.0, tied_head=True,
+                             mixers=(("attention", "conv_attention"),))}
 NO_POS_LIMIT = 1 << 30
 
 
@@ -322,7 +338,8 @@ class Mixer:
         raise NotImplementedError
 
     def cache_spec(self):
-        """("paged", width) | ("state", {name: shape}) | a list of those | None."""
+        """("paged", width) | ("pooled", (width, every)) | ("state", {name: shape}) | a list of
+        those | None."""
         return None
 
     # A mixer either implements ``forward`` (it projects its input itself), or exposes the
@@ -332,6 +349,7 @@ class Mixer:
     w_in = None
     b_in = None   # bias of the input product (activation type), or None
     wo = None
+    b_out = None  # bias of the output product (activation type), or None
     n_mid = 0
 
     def mix(self, proj, b: "StepBatch", cache, layer: int, out, out_scale: float = 1.0):
@@ -340,7 +358,7 @@ class Mixer:
 
     def forward_proj(self, proj, b: "StepBatch", cache, layer: int):
         mid = torch.empty(b.R, self.n_mid, device=proj.device, dtype=proj.dtype)
-        return F.linear(self.mix(proj, b, cache, layer, mid), self.wo)
+        return F.linear(self.mix(proj, b, cache, layer, mid), self.wo, self.b_out)
 
     def forward(self, h, b: "StepBatch", cache, layer: int):
         return self.forward_proj(F.linear(h, self.w_in, self.b_in), b, cache, layer)
@@ -429,6 +447,92 @@ class Mamba2(Mixer):
         yn = torch.empty(b.R, self.inner, device=h.device, dtype=h.dtype)
         sm.rmsnorm(y, self.normw, self.eps, yn, parts=self.ng)
         return F.linear(yn, self.wo)
+
+
+class Mamba1(Mixer):
+    """The first Mamba (``ops.seqmix.selective_scan``): W_in gives x and a gate z, x passes a short
+    convolution + silu; step sizes (through a rank of ``dt_rank``), B and C are projections of it;
+    every channel carries ``state`` numbers with decays of their own."""
+    kind = "mamba1"
+
+    def _dims(self):
+        s = self.spec
+        self.I, self.N, self.rank, self.K = (int(s[k]) for k in ("inner", "state", "dt_rank", "conv"))
+        if min(self.I, self.N, self.rank, self.K) < 1:
+            raise ValueError("mamba1: inner %d / state %d / rank %d / %d taps" % (self.I, self.N, self.rank, self.K))
+        self.n_mid = self.I
+
+    def tensor_shapes(self):
+        self._dims()
+        I, N, r, W = self.I, self.N, self.rank, self.width
+        return {"in": (2 * I, W), "conv": (I, self.K), "conv.b": (I,), "x": (r + 2 * N, I), "dt": (I, r),
+                "dt.b": (I,), "A_log": (I, N), "D": (I,), "o": (W, I)}
+
+    def load(self, get, dtype, dev):
+        self._dims()
+        self.w_in = get("in").to(dev, dtype).contiguous()
+        self.cw, self.cb = _vec(get("conv"), dev), _vec(get("conv.b"), dev)
+        self.w_x = get("x").to(dev, dtype).contiguous()
+        self.w_dt = get("dt").to(dev, dtype).t().contiguous()                     # [rank, I]
+        self.dtb, self.Dp = _vec(get("dt.b"), dev), _vec(get("D"), dev)
+        # A = -exp(A_log) as a base-2 exponent, states by rows
+        self.A2 = (-torch.exp(get("A_log").double()) * sm.LOG2E).t().float().contiguous().to(dev)
+        self.wo = get("o").to(dev, dtype).contiguous()
+
+    def cache_spec(self):
+        return ("state", {"S": (self.N, self.I), "tail": (self.K - 1, self.I)})
+
+    def mix(self, proj, b, cache, layer, out, out_scale=1.0):
+        st, I = cache.state[layer], self.I
+        x = torch.empty(b.R, I, device=proj.device, dtype=proj.dtype)
+        sm.mamba_conv(proj, 0, self.cw, self.cb, st["tail"], b.ent, b.ent_host, b.row_ent, x, roll=True)
+        xp = F.linear(x, self.w_x)
+        sm.selective_scan(x, xp, self.rank, self.w_dt, self.dtb, self.A2, self.Dp, proj[:, I:2 * I],
+                          st["S"], b.ent, b.ent_host, out)
+        if out_scale != 1.0:
+            out.mul_(out_scale)
+        return out
+
+
+class Lightning(Mixer):
+    """Linear attention with a constant decay per head (``ops.seqmix.lightning_scan``): silu on q, k
+    and v, one RMS norm over all heads with a weight per channel, a sigmoid gate per channel."""
+    kind = "lightning"
+
+    def _dims(self):
+        s = self.spec
+        self.H, self.D, self.V = int(s["heads"]), int(s["dim"]), int(s["vdim"])
+        self.decay = [float(x) for x in s["decay"]]
+        if len(self.decay) != self.H:
+            raise ValueError("lightning: %d decays for %d heads" % (len(self.decay), self.H))
+        self.n_mid = self.H * self.V
+
+    def tensor_shapes(self):
+        self._dims()
+        H, D, V, W = self.H, self.D, self.V, self.width
+        return {"q": (H * D, W), "k": (H * D, W), "v": (H * V, W), "g": (H * V, W), "o": (W, H * V),
+                "norm": (H * V,)}
+
+    def load(self, get, dtype, dev):
+        self._dims()
+        # one projection for everything that reads the layer input: q | k | v | gate
+        self.w_in = torch.cat([get(k) for k in ("q", "k", "v", "g")], 0).to(dev, dtype).contiguous()
+        self.lam = torch.tensor(self.decay, dtype=torch.float32, device=dev)
+        self.normw = _vec(get("norm"), dev)
+        self.wo = get("o").to(dev, dtype).contiguous()
+
+    def cache_spec(self):
+        return ("state", {"S": (self.H, self.D, self.V)})
+
+    def mix(self, proj, b, cache, layer, out, out_scale=1.0):
+        H, D, V = self.H, self.D, self.V
+        o = torch.empty(b.R, H * V, device=proj.device, dtype=torch.float32)
+        sm.lightning_scan(proj, self.lam, cache.state[layer]["S"], b.ent, b.ent_host, o, H, D, V)
+        g0 = 2 * H * D + H * V
+        sm.norm_gate(o, self.normw, proj[:, g0:g0 + H * V], self.eps, out)
+        if out_scale != 1.0:
+            out.mul_(out_scale)
+        return out
 
 
 class LatentAttention(Mixer):
@@ -609,6 +713,72 @@ class BiasedAttention(Mixer):
         sm.window_attn(q, pool, b.block_tables, b.row_ent, b.pos, self.sink, self.scale, self.win,
                        out, PAGE, H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale,
                        softcap=self.cap, dist=(self.r1, self.r2), gate=proj[:, nq + nkv:])
+        return out
+
+
+class ConvAttention(Mixer):
+    """Grouped-query attention behind short convolutions (``ops.seqmix.conv_rope_norm_store``,
+    ``window_attn``): biased q / k / v projections, a causal convolution of ``conv`` taps on each of
+    their channels, rotation of the pairs (i, i + dims/2), query and key heads divided by their root
+    mean square, scores times ``scale`` and a learned factor per head.  ``mask.size`` is a sliding
+    window (optional); with ``mask.pool`` every block of that many tokens that lies wholly before
+    the window is seen as one key and value, the means of its tokens' as the cache holds them.
+    The result leaves through a sigmoid gate per channel and a biased output projection."""
+    kind = "conv_attention"
+
+    def _dims(self):
+        s = self.spec
+        self.H, self.D, self.V = int(s["heads"]), int(s["dim"]), int(s["vdim"])
+        self.G, self.K = int(s.get("kv_heads", self.H)), int(s["conv"])
+        mask = s.get("mask") or {}
+        self.win = int(mask.get("size", 1 << 30))
+        self.pool = int(mask.get("pool") or 0)
+        self.scale = float(s["scale"]) if "scale" in s else self.D ** -0.5
+        rot = s.get("rot")
+        self.rot_dims, self.rot_base = (int(rot["dims"]), float(rot["base"])) if rot else (0, 1.0)
+        if self.H % self.G or self.rot_dims % 2 or self.rot_dims > self.D or self.K < 1 or self.win < 1 \
+                or self.pool < 0:
+            raise ValueError("conv_attention: %d heads / %d kv heads / %d rotated of %d channels / %d taps / "
+                             "window %d / blocks of %d" % (self.H, self.G, self.rot_dims, self.D, self.K,
+                                                           self.win, self.pool))
+        self.n_mid = self.H * self.V
+        self.C = (self.H + self.G) * self.D + self.G * self.V
+
+    def tensor_shapes(self):
+        self._dims()
+        H, G, D, V, W = self.H, self.G, self.D, self.V, self.width
+        d = {"temp": (H,), "g": (H * V, W), "o": (W, H * V), "o.b": (W,)}
+        for k, n in (("q", H * D), ("k", G * D), ("v", G * V)):
+            d.update({k: (n, W), k + ".b": (n,), k + ".conv": (n, self.K)})
+        return d
+
+    def load(self, get, dtype, dev):
+        self._dims()
+        # one projection for everything that reads the layer input: q | k | v | gate
+        self.w_in = torch.cat([get(k) for k in ("q", "k", "v", "g")], 0).to(dev, dtype).contiguous()
+        self.b_in = torch.cat([get("q.b"), get("k.b"), get("v.b"),
+                               torch.zeros(self.n_mid, dtype=get("q.b").dtype)]).to(dev, dtype).contiguous()
+        self.cw = torch.cat([_vec(get(k), dev) for k in ("q.conv", "k.conv", "v.conv")], 0).contiguous()
+        self.temp = _vec(get("temp"), dev)
+        self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev)
+        self.wo, self.b_out = (get(k).to(dev, dtype).contiguous() for k in ("o", "o.b"))
+
+    def cache_spec(self):
+        w = self.G * (self.D + self.V)
+        return [("paged", w), ("state", {"tail": (self.K - 1, self.C)})] + \
+            ([("pooled", (w, self.pool))] if self.pool else [])
+
+    def mix(self, proj, b, cache, layer, out, out_scale=1.0):
+        H, G, D, V = self.H, self.G, self.D, self.V
+        pool, blk = cache.paged[layer], cache.pooled.get(layer)
+        q = torch.empty(b.R, H * D, device=proj.device, dtype=proj.dtype)
+        sm.conv_rope_norm_store(proj, H, G, D, V, self.cw, cache.state[layer]["tail"], self.inv_freq,
+                                self.temp, b.pos, b.cache_rows, pool, self.eps, q, b.ent, b.ent_host,
+                                b.row_ent, b.block_tables, PAGE, blk=blk, every=self.pool)
+        units = b.units(sm.window_rows_per_wave(H // G)) if sm.window_mfma_ok(q, pool, D, V) else None
+        sm.window_attn(q, pool, b.block_tables, b.row_ent, b.pos, None, self.scale, self.win, out, PAGE,
+                       H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale,
+                       gate=proj[:, self.C:], gate_channels=True, blk=blk, every=self.pool)
         return out
 
 
@@ -862,7 +1032,8 @@ class Parallel(Mixer):
 
 
 MIXERS = {c.kind: c for c in (GeneralDelta, Mamba2, LatentAttention, WindowAttention, GatedDelta,
-                              HGRN2, Parallel, Attention, MLSTM, BiasedAttention, RopeLatentAttention)}
+                              HGRN2, Parallel, Attention, MLSTM, BiasedAttention, RopeLatentAttention,
+                              ConvAttention, Mamba1, Lightning)}
 
 
 class DenseFF:
@@ -1161,6 +1332,13 @@ class HybridLayer:
                 d["norm2"] = ()
                 d.update({"mlp." + k: s for k, s in self.ff.tensor_shapes().items()})
             return d
+        if self.block == "post":
+            d = {"norm1": (W,)}
+            d.update({"mix." + k: s for k, s in self.mixer.tensor_shapes().items()})
+            if self.ff is not None:
+                d["norm2"] = (W,)
+                d.update({"mlp." + k: s for k, s in self.ff.tensor_shapes().items()})
+            return d
         if self.block == "parallel":
             d = {"norm1": (W,)}
             d.update({"mix." + k: s for k, s in self.mixer.tensor_shapes().items()})
@@ -1194,6 +1372,11 @@ class HybridLayer:
                     outs.append(self.ff.w_out)
             self.w_out_all = torch.cat(outs, 1).contiguous() if len(outs) > 1 else outs[0]
             return
+        if self.block == "post":
+            self.norm1 = (_vec(sd[p + "norm1"], dev) + self.norm_offset).contiguous()
+            if self.ff is not None:
+                self.norm2 = (_vec(sd[p + "norm2"], dev) + self.norm_offset).contiguous()
+            return
         if self.block == "parallel":
             if self.mixer.w_in is None or self.mixer.wo is None:
                 raise ValueError("mixer %r cannot share the layer's products" % self.mixer.kind)
@@ -1225,8 +1408,9 @@ class HybridLayer:
 def tensor_shapes(cfg: HybridConfig) -> dict:
     """name -> shape of every tensor of a checkpoint of this config."""
     W = cfg.width
-    d = {"embed": (cfg.vocab, W), "final.norm": () if cfg.traits.scalar_norms else (W,),
-         "head": (cfg.vocab, W)}
+    d = {"embed": (cfg.vocab, W), "final.norm": () if cfg.traits.scalar_norms else (W,)}
+    if not cfg.traits.tied_head:
+        d["head"] = (cfg.vocab, W)
     if cfg.traits.positions:
         d["pos"] = (cfg.max_pos, W)
     if cfg.loop:
@@ -1254,7 +1438,7 @@ class HybridWeights:
         self.pos = sd["pos"].to(dev, dtype).contiguous() if cfg.traits.positions else None
         self.final_norm = (_vec(sd["final.norm"], dev) + cfg.traits.norm_offset).expand(cfg.width).contiguous() \
             if cfg.traits.scalar_norms else (_vec(sd["final.norm"], dev) + cfg.traits.norm_offset).contiguous()
-        self.head = sd["head"].to(dev, dtype).contiguous()
+        self.head = self.embed if cfg.traits.tied_head else sd["head"].to(dev, dtype).contiguous()
         self.loop_step = _vec(sd["loop.step"], dev) if cfg.loop else None
         self.layers = []
         for i, spec in enumerate(cfg.layers):
@@ -1312,6 +1496,10 @@ def random_state_dict(cfg: HybridConfig, seed: int = 0) -> dict:
             t = torch.rand(*s, generator=g) * (2.0 if leaf.endswith("r1") else 0.3)
         elif k == "loop.step":
             t = torch.randn(*s, generator=g) * 0.5
+        elif leaf.endswith("mix.dt.b"):
+            t = torch.randn(*s, generator=g) - 2.0
+        elif leaf.endswith("mix.temp"):
+            t = 1.0 + 0.2 * torch.randn(*s, generator=g)
         elif leaf.endswith(("dt_bias", "mix.D")):
             t = torch.randn(*s, generator=g) * 0.5
         else:
@@ -1351,6 +1539,8 @@ class HybridModel:
             return self._forward_parallel(b, layer_out)
         if cfg.traits.block == "parallel2":
             return self._forward_parallel2(b, layer_out)
+        if cfg.traits.block == "post":
+            return self._forward_post(b, layer_out)
         x = torch.empty(b.R, cfg.width, device=self.device, dtype=torch.float32)
         sm.embed_pos(w.embed, w.pos, b.ids, b.pos, x)
         h = torch.empty(b.R, cfg.width, device=self.device, dtype=self.dtype)
@@ -1360,11 +1550,12 @@ class HybridModel:
         for i, L in enumerate(w.layers):
             after = w.layers[i + 1].norm1 if i + 1 < len(w.layers) else None
             m = L.mixer.forward(h, b, self.cache, i)
-            sm.norm_scale_add(x, m, L.norm1b, L.ls1, cfg.eps,
-                              next_w=L.norm2 if L.ff is not None else after, next_out=h)
+            nxt = L.norm2 if L.ff is not None else after
+            sm.norm_scale_add(x, m, L.norm1b, L.ls1, cfg.eps, next_w=nxt,
+                              next_out=h if nxt is not None else None)
             if L.ff is not None:
                 sm.norm_scale_add(x, L.ff.forward(h), L.norm2b, L.ls2, cfg.eps, next_w=after,
-                                  next_out=h)
+                                  next_out=h if after is not None else None)
             if layer_out is not None:
                 layer_out.append(x.clone())
         if b.n_out == 0:
@@ -1455,6 +1646,28 @@ class HybridModel:
                     n = L.ff.w_in.shape[0]
                     f, gate = L.ff.forward_proj(proj[:, :n]), proj[:, n:]
                 sm.gate_norm_add(x, f, gate, L.rg2b, L.norm2, parts, eps, next_out=nxt)
+            if layer_out is not None:
+                layer_out.append(x.clone())
+        if b.n_out == 0:
+            return None
+        return self._logits(x, b)
+
+    def _forward_post(self, b: StepBatch, layer_out=None):
+        """x <- x + N(f(x)) per sublayer: a sublayer reads the residual rows themselves (rounded to the
+        activation type), and the pass that norms and adds what it produced also writes them for
+        the next one."""
+        cfg, w = self.cfg, self.w
+        x = torch.empty(b.R, cfg.width, device=self.device, dtype=torch.float32)
+        # in float32 the sublayers read the residual stream itself
+        h = x if self.dtype == torch.float32 else \
+            torch.empty(b.R, cfg.width, device=self.device, dtype=self.dtype)
+        nxt = None if h is x else h
+        sm.embed_rows(w.embed, b.ids, x, nxt, scale=cfg.embed_scale)
+        for i, L in enumerate(w.layers):
+            m = L.mixer.forward(h, b, self.cache, i)
+            sm.norm_scale_add(x, m, L.norm1, None, cfg.eps, next_out=nxt)
+            if L.ff is not None:
+                sm.norm_scale_add(x, L.ff.forward(h), L.norm2, None, cfg.eps, next_out=nxt)
             if layer_out is not None:
                 layer_out.append(x.clone())
         if b.n_out == 0:

@@ -1,10 +1,12 @@
-"""Sequence-mixer ops: recurrent state layers (generalized delta rule, Mamba-2, gated delta
-rule, HGRN2, the mLSTM's matrix memory), latent attention (optionally with a rotated key part
+"""Sequence-mixer ops: recurrent state layers (generalized delta rule, Mamba-2, the selective
+scan of the first Mamba, gated delta rule, HGRN2, lightning attention, the mLSTM's matrix memory),
+latent attention (optionally with a rotated key part
 in the cached row and without a sink) and grouped-query attention with an optional sliding
 window and softmax sink (query/key norm over the row or per head, rotary positions on adjacent
 or half-split channel pairs and the cache write in one pass; or unrotated with a query
-temperature, capped scores, a logarithmic distance penalty and a gate per head), a
-group-limited expert router (sigmoid or softmax scores, optional score correction and bias,
+temperature, capped scores, a logarithmic distance penalty and a gate per head; or behind short
+convolutions, with unit-RMS heads, pooled blocks of the tokens before the window and a gate per
+channel), a group-limited expert router (sigmoid or softmax scores, optional score correction and bias,
 softmax over the chosen logits) with grouped expert products and identity experts, learned
 positions, and the norms, residual passes (one with two normed outputs and the routed experts'
 weighted sum) and pointwise steps around them.
@@ -53,12 +55,30 @@ _SIGS = {
                                   c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int,
                                   c_int, c_void_p],
     "p2p_sm_mamba_conv": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
-                          c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+                          c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                          c_void_p],
+    "p2p_sm_norm_gate": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
+                         c_float, c_int, c_void_p],
+    "p2p_sm_selective_scan": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
+                              c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                              c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
+                              c_void_p],
+    "p2p_sm_selective_step": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
+                              c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
+                              c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    "p2p_sm_lightning_scan": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                              c_int, c_int, c_int, c_int, c_void_p],
+    "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
+                                    c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
+                                    c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                                    c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    "p2p_sm_pool_blocks": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
+                           c_int, c_int, c_void_p],
     "p2p_sm_mamba_scan": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int,
                           c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_mamba_tail": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                          c_void_p],
+                          c_int, c_void_p],
     "p2p_sm_latent_attn": [c_void_p, c_long, c_long, c_void_p, c_void_p, c_int, c_void_p,
                            c_void_p, c_void_p, c_float, c_int, c_void_p, c_long, c_long, c_int,
                            c_int, c_int, c_int, c_int, c_void_p],
@@ -100,11 +120,12 @@ _SIGS = {
     "p2p_sm_window_attn": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                            c_void_p, c_float, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
                            c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int,
-                           c_int, c_void_p],
+                           c_int, c_void_p, c_int, c_int, c_void_p],
     "p2p_sm_window_attn_mfma": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                                 c_void_p, c_int, c_void_p, c_float, c_int, c_void_p, c_int, c_int,
                                 c_int, c_int, c_int, c_int, c_int, c_void_p, c_float, c_float,
-                                c_void_p, c_void_p, c_void_p, c_int, c_void_p],
+                                c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int,
+                                c_void_p],
     "p2p_sm_hgrn2_scan": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                           c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
                           c_void_p],
@@ -282,16 +303,16 @@ def rmsnorm(x, w, eps, out, parts: int = 1, in_rows=None, out_rows=None):
 
 def norm_scale_add(x, y, w, ls, eps, next_w=None, next_out=None):
     """x += y / sqrt(mean(y^2) + eps) * w * ls on the fp32 residual x (ls may be None).
-    With next_w / next_out also the next sublayer's input in the same pass:
-    next_out = x / sqrt(mean(x^2) + eps) * next_w from the updated rows."""
+    With next_out also the next sublayer's input in the same pass, from the updated rows:
+    next_out = x / sqrt(mean(x^2) + eps) * next_w, or without next_w the rows as they are."""
     R, n = x.shape
     if not x.is_cuda:
         v = _rms(y.float(), eps) * w
         if ls is not None:
             v = v * ls
         x += v
-        if next_w is not None:
-            next_out[:R] = (_rms(x, eps) * next_w).to(next_out.dtype)
+        if next_out is not None:
+            next_out[:R] = (_rms(x, eps) * next_w if next_w is not None else x).to(next_out.dtype)
         return x
     _rows2d(y, "y")
     assert x.dtype == torch.float32 and x.is_contiguous() and y.shape == x.shape
@@ -301,12 +322,13 @@ def norm_scale_add(x, y, w, ls, eps, next_w=None, next_out=None):
     ldh = 0
     if next_w is not None:
         _vec(next_w, n, "next_w")
+    if next_out is not None:
         _rows2d(next_out, "next_out")
         assert next_out.dtype == y.dtype and next_out.shape[1] == n and next_out.shape[0] >= R
         ldh = next_out.stride(0)
     _chk(lib().p2p_sm_norm_scale_add(x.data_ptr(), y.data_ptr(), y.stride(0), w.data_ptr(),
                                      _lib.ptr(ls), R, n, eps, _lib.ptr(next_w),
-                                     _lib.ptr(next_out if next_w is not None else None), ldh,
+                                     _lib.ptr(next_out), ldh,
                                      _f32(y), _st(x)), "norm_scale_add")
     return x
 
@@ -415,6 +437,24 @@ def add_norm2(x, a=None, b=None, rows=None, vec=None, eps: float = 0.0, w1=None,
                                 _f32(act) if act is not None else 1, _st(x)),
          "add_norm2")
     return x
+
+
+def norm_gate(x, w, g, eps, out):
+    """out = x / sqrt(mean(x^2) + eps) * w * sigmoid(g): x fp32 [R, n], w fp32 [n], g and out
+    activation-typed [R, n]."""
+    R, n = x.shape
+    if not x.is_cuda:
+        out[:R] = (_rms(x, eps) * w * torch.sigmoid(g[:R, :n].float())).to(out.dtype)
+        return out
+    for t_, nm in ((x, "x"), (g, "g"), (out, "out")):
+        _rows2d(t_, nm)
+        assert t_.shape[0] >= R and t_.shape[1] == n, nm
+    assert x.dtype == torch.float32 and g.dtype == out.dtype
+    _vec(w, n, "w")
+    _chk(lib().p2p_sm_norm_gate(x.data_ptr(), x.stride(0), w.data_ptr(), g.data_ptr(), g.stride(0),
+                                out.data_ptr(), out.stride(0), R, n, eps, _f32(out), _st(x)),
+         "norm_gate")
+    return out
 
 
 # ------------------------------------------------------------------ pointwise
@@ -547,10 +587,12 @@ def gdelta_scan(r, k, v, g, a, lo, w0, ab, normw, state, ent, ent_host, out, H: 
 
 
 # ------------------------------------------------------------------ Mamba-2
-def mamba_conv(zx, xoff: int, cw, cb, tail, ent, ent_host, row_ent, out):
+def mamba_conv(zx, xoff: int, cw, cb, tail, ent, ent_host, row_ent, out, roll: bool = False):
     """Causal per-channel convolution + bias + silu over channels [xoff, xoff + C) of zx.
     cw fp32 [C, K] (column K-1 multiplies the newest input), tail fp32 [slots, K-1, C] the raw inputs
-    before each slot's next token (read only here; ``mamba_scan`` rolls it)."""
+    before each slot's next token; out [R, C] fp32 or activation typed.  roll: the tails move
+    forward as well (in the same kernel for portions of one token, ``conv_tail_roll`` for the
+    others); without it they are only read (``mamba_scan`` / ``conv_tail_roll`` follow)."""
     R, C = out.shape
     K = cw.shape[1]
     if not zx.is_cuda:
@@ -561,29 +603,37 @@ def mamba_conv(zx, xoff: int, cw, cb, tail, ent, ent_host, row_ent, out):
             acc = cb.clone().expand(n, C).clone()
             for kk in range(K):
                 acc += pad[kk:kk + n] * cw[:, kk]
-            out[row0:row0 + n] = acc * torch.sigmoid(acc)
+            out[row0:row0 + n] = (acc * torch.sigmoid(acc)).to(out.dtype)
+        if roll:
+            conv_tail_roll(zx, xoff, tail, ent, ent_host, C)
         return out
     _rows2d(zx, "zx")
-    assert out.dtype == torch.float32 and out.is_contiguous()
+    _rows2d(out, "out")
+    assert out.dtype in (torch.float32, zx.dtype)
     assert cw.dtype == torch.float32 and cw.is_contiguous() and cw.shape[0] == C
     _vec(cb, C, "cb")
     assert tail.dtype == torch.float32 and tail.is_contiguous() and tail.shape[1:] == (K - 1, C)
     assert xoff + C <= zx.shape[1] and row_ent.dtype == torch.int32
     _chk(lib().p2p_sm_mamba_conv(zx.data_ptr(), zx.stride(0), xoff, cw.data_ptr(), cb.data_ptr(),
                                  tail.data_ptr(), ent.data_ptr(), row_ent.data_ptr(),
-                                 out.data_ptr(), R, C, K, _f32(zx), _st(zx)), "mamba_conv")
+                                 out.data_ptr(), out.stride(0), _f32(out), R, C, K,
+                                 1 if roll else 0, _f32(zx), _st(zx)), "mamba_conv")
+    if roll:
+        conv_tail_roll(zx, xoff, tail, ent, ent_host, C, skip_single=True)
     return out
 
 
-def conv_tail_roll(zx, xoff: int, tail, ent, ent_host, C: int):
+def conv_tail_roll(zx, xoff: int, tail, ent, ent_host, C: int, skip_single: bool = False):
     """After a step's convolutions: every entry's slot keeps the raw inputs (channels
     [xoff, xoff + C) of zx) of its last K-1 tokens, older ones shifted out.  tail fp32
-    [slots, K-1, C]."""
+    [slots, K-1, C].  skip_single: entries of one token have been dealt with."""
     Km1 = tail.shape[1]
-    if Km1 == 0:
+    if Km1 == 0 or (skip_single and all(e[1] == 1 for e in ent_host)):
         return tail
     if not zx.is_cuda:
         for row0, n, start, slot in ent_host:
+            if skip_single and n == 1:
+                continue
             raw = zx[row0:row0 + n, xoff:xoff + C].float()
             prev = tail[slot] if start > 0 else torch.zeros(Km1, C)
             tail[slot] = torch.cat([prev, raw], 0)[-Km1:]
@@ -592,7 +642,8 @@ def conv_tail_roll(zx, xoff: int, tail, ent, ent_host, C: int):
     assert tail.dtype == torch.float32 and tail.is_contiguous() and tail.shape[2] == C
     assert xoff + C <= zx.shape[1]
     _chk(lib().p2p_sm_mamba_tail(zx.data_ptr(), zx.stride(0), xoff, tail.data_ptr(),
-                                 ent.data_ptr(), ent.shape[0], C, Km1 + 1, _f32(zx), _st(zx)),
+                                 ent.data_ptr(), ent.shape[0], C, Km1 + 1,
+                                 1 if skip_single else 0, _f32(zx), _st(zx)),
          "conv_tail_roll")
     return tail
 
@@ -654,7 +705,72 @@ def mamba_scan(conv, zx, xoff: int, dtoff: int, dt_bias, A_log, Dp, state, tail,
                                      y.data_ptr(), H, P, N, G, Km1 + 1, _f32(zx), _st(zx)),
              "mamba_scan")
     _chk(lib().p2p_sm_mamba_tail(zx.data_ptr(), zx.stride(0), xoff, tail.data_ptr(),
-                                 ent.data_ptr(), E, C, Km1 + 1, _f32(zx), _st(zx)), "mamba_tail")
+                                 ent.data_ptr(), E, C, Km1 + 1, 0, _f32(zx), _st(zx)), "mamba_tail")
+    return y
+
+
+# ------------------------------------------------------------------ selective scan (Mamba)
+LOG2E = math.log2(math.e)
+
+
+def selective_scan(x, xp, rank: int, wdt, dt_bias, A2, Dp, z, state, ent, ent_host, y):
+    """Selective state-space scan of the first Mamba, I channels with N states of their own.
+    x [R, I] the convolved inputs, xp = [low-rank step sizes (rank) | B (N) | C (N)] per row, z [R, I]
+    the gate, all activation typed.  dt = softplus(wdt^T low + dt_bias) with wdt [rank, I]
+    (activation type); A2 fp32 [N, I] = A * log2(e);
+        S[n, c] <- exp(dt_c A[n, c]) S[n, c] + dt_c x_c B_n,   y_c = (sum_n S[n, c] C_n + D_c x_c) silu(z_c).
+    state fp32 [slots, N, I]; y [R, I] activation type.  A step of single tokens runs one fused
+    kernel per row (projection of dt included); portions project dt with one product first, and
+    long ones are scanned in chunks."""
+    R, I = y.shape
+    N = A2.shape[0]
+    assert xp.shape[1] == rank + 2 * N and wdt.shape == (rank, I)
+    if not x.is_cuda:
+        A = A2 / LOG2E
+        low = torch.nn.functional.softplus(xp[:, :rank].float() @ wdt.float() + dt_bias, threshold=1e9)
+        for row0, n, start, slot in ent_host:
+            S = state[slot] if start > 0 else torch.zeros_like(state[slot])
+            for t in range(row0, row0 + n):
+                xv, dt = x[t].float(), low[t]
+                S = torch.exp(dt * A) * S + (dt * xv)[None, :] * xp[t, rank:rank + N].float()[:, None]
+                zz = z[t].float()
+                yy = xp[t, rank + N:].float() @ S + Dp * xv
+                y[t] = (yy * (zz * torch.sigmoid(zz))).to(y.dtype)
+            state[slot] = S
+        return y
+    for t_, nm in ((x, "x"), (xp, "xp"), (z, "z"), (y, "y")):
+        _rows2d(t_, nm)
+        assert t_.dtype == y.dtype and t_.shape[0] >= R, nm
+    assert x.shape[1] == I and z.shape[1] == I and wdt.dtype == y.dtype and wdt.is_contiguous()
+    _vec(dt_bias, I, "dt_bias")
+    _vec(Dp, I, "D")
+    assert A2.dtype == torch.float32 and A2.is_contiguous() and A2.shape == (N, I)
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (N, I)
+    assert ent.dtype == torch.int32 and ent.is_contiguous() and ent.shape[1] == 4
+    if N > 512:
+        raise ValueError("selective_scan: %d states per channel > 512" % N)
+    E = ent.shape[0]
+    bc = xp[:, rank:]
+    if all(e[1] == 1 for e in ent_host):
+        _chk(lib().p2p_sm_selective_step(
+            x.data_ptr(), x.stride(0), bc.data_ptr(), xp.stride(0), xp.data_ptr(), xp.stride(0),
+            wdt.data_ptr(), rank, dt_bias.data_ptr(), A2.data_ptr(), Dp.data_ptr(), z.data_ptr(),
+            z.stride(0), state.data_ptr(), ent.data_ptr(), E, y.data_ptr(), y.stride(0), I, N,
+            _f32(y), _st(y)), "selective_step")
+        return y
+    dt = torch.mm(xp[:, :rank], wdt)
+    vent = cent = tmp = dtsum = None
+    NV = 0
+    if _chunked(ent_host):
+        vent, cent = (t_.to(y.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        NV = vent.shape[0]
+        tmp = torch.empty(NV, N, I, device=y.device, dtype=torch.float32)
+        dtsum = torch.empty(NV, I, device=y.device, dtype=torch.float32)
+    _chk(lib().p2p_sm_selective_scan(
+        x.data_ptr(), x.stride(0), bc.data_ptr(), xp.stride(0), dt.data_ptr(), dt.stride(0),
+        dt_bias.data_ptr(), A2.data_ptr(), Dp.data_ptr(), z.data_ptr(), z.stride(0),
+        state.data_ptr(), ent.data_ptr(), E, y.data_ptr(), y.stride(0), I, N, _lib.ptr(vent), NV,
+        _lib.ptr(cent), _lib.ptr(tmp), _lib.ptr(dtsum), _f32(y), _st(y)), "selective_scan")
     return y
 
 
@@ -1030,6 +1146,95 @@ def qk_norm_rope_store(proj, H: int, G: int, D: int, V: int, qw, kw, inv_freq, p
     return q_out
 
 
+def blocks_per_page(page: int, every: int) -> int:
+    """Rows a page has in a pool of blocks of ``every`` tokens: the most blocks that end in it."""
+    return -(-page // every)
+
+
+def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_freq, temp, pos,
+                         cache_rows, pool, eps: float, q_out, ent, ent_host, row_ent,
+                         block_tables, page: int, blk=None, every: int = 0):
+    """Prepares attention inputs from one projection buffer proj = [q (H*D) | k (G*D) | v (G*V) | ..]:
+    every channel goes through a causal convolution over time (cw fp32 [C, K], column K-1 the newest
+    input, no bias; tail fp32 [slots, K-1, C] the projections before each slot's next token, moved
+    forward here), the pairs (i, i + nrot), i < nrot = len(inv_freq), of every q and k head are turned
+    by pos * inv_freq[i], q and k heads are divided by sqrt(mean(x^2) + eps), and q head h is multiplied
+    by temp[h] (fp32 [H] or None).  q goes to q_out [R, H*D], k | v to the rows ``cache_rows`` of the
+    paged pool.  All of it fp32.
+    blk: a pool of blocks of ``every`` tokens ([pages * blocks_per_page, G*(D+V)]); the blocks that
+    this step's tokens complete get the mean of their tokens' rows of ``pool``."""
+    R = q_out.shape[0]
+    nq, nk, nv = H * D, G * D, G * V
+    C, K = nq + nk + nv, cw.shape[1]
+    nrot = inv_freq.numel()
+    sb = blocks_per_page(page, every) if blk is not None else 0
+    if not proj.is_cuda:
+        y = torch.empty(R, C)
+        for row0, n, start, slot in ent_host:
+            prev = tail[slot] if start > 0 else torch.zeros(K - 1, C)
+            pad = torch.cat([prev, proj[row0:row0 + n, :C].float()], 0)
+            y[row0:row0 + n] = sum(pad[kk:kk + n] * cw[:, kk] for kk in range(K))
+        conv_tail_roll(proj, 0, tail, ent, ent_host, C)
+        ang = pos[:R].float()[:, None] * inv_freq[None, :]
+        c, sn = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+
+        def prep(t, heads):
+            t = t.reshape(R, heads, D).clone()
+            u, w = t[:, :, :nrot].clone(), t[:, :, nrot:2 * nrot].clone()
+            t[:, :, :nrot] = u * c - w * sn
+            t[:, :, nrot:2 * nrot] = w * c + u * sn
+            return _rms(t, eps)
+
+        q = prep(y[:, :nq], H)
+        if temp is not None:
+            q = q * temp[:, None]
+        q_out[:R] = q.reshape(R, nq).to(q_out.dtype)
+        rows = cache_rows[:R].long()
+        pool[rows, :nk] = prep(y[:, nq:nq + nk], G).reshape(R, nk).to(pool.dtype)
+        pool[rows, nk:] = y[:, nq + nk:].to(pool.dtype)
+        if blk is not None:
+            bt = block_tables.long()
+            for e, (row0, n, start, slot) in enumerate(ent_host):
+                for b in range(start // every, (start + n) // every):
+                    j = torch.arange(b * every, b * every + every)
+                    last = int(j[-1])
+                    blk[int(bt[e][last // page]) * sb + last % page // every] = \
+                        pool[bt[e][j // page] * page + j % page].float().mean(0).to(blk.dtype)
+        return q_out
+    _rows2d(proj, "proj")
+    _rows2d(q_out, "q_out")
+    assert proj.shape[1] >= C and q_out.shape[1] == nq and q_out.dtype == proj.dtype
+    assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == nk + nv and pool.dtype == proj.dtype
+    assert cw.dtype == torch.float32 and cw.is_contiguous() and cw.shape[0] == C
+    assert tail.dtype == torch.float32 and tail.is_contiguous() and tail.shape[1:] == (K - 1, C)
+    assert inv_freq.dtype == torch.float32 and inv_freq.is_contiguous() and 2 * nrot <= D
+    assert pos.dtype == torch.int32 and cache_rows.dtype == torch.int32 and row_ent.dtype == torch.int32
+    assert ent.dtype == torch.int32 and ent.is_contiguous() and ent.shape[1] == 4
+    assert block_tables.dtype == torch.int32 and block_tables.is_contiguous()
+    if temp is not None:
+        _vec(temp, H, "temp")
+    if blk is not None:
+        assert every >= 1 and blk.is_contiguous() and blk.dtype == pool.dtype
+        assert blk.shape == (pool.shape[0] // page * sb, pool.shape[1])
+    if 4 * max(D, V) * 4 > 64 * 1024:
+        raise ValueError("conv_rope_norm_store: head sizes %d / %d" % (D, V))
+    _chk(lib().p2p_sm_conv_rope_norm_store(
+        proj.data_ptr(), proj.stride(0), H, G, D, V, cw.data_ptr(), K, tail.data_ptr(),
+        ent.data_ptr(), row_ent.data_ptr(), inv_freq.data_ptr(), nrot, _lib.ptr(temp), eps,
+        pos.data_ptr(), cache_rows.data_ptr(), pool.data_ptr(), q_out.data_ptr(), q_out.stride(0),
+        _lib.ptr(blk), every, block_tables.data_ptr(), block_tables.shape[1], page, R, _f32(proj),
+        _st(proj)), "conv_rope_norm_store")
+    conv_tail_roll(proj, 0, tail, ent, ent_host, C, skip_single=True)
+    if blk is not None:
+        most = max([(e[2] + e[1]) // every - e[2] // every for e in ent_host if e[1] > 1] or [0])
+        if most:
+            _chk(lib().p2p_sm_pool_blocks(pool.data_ptr(), pool.shape[1], blk.data_ptr(), every,
+                                          ent.data_ptr(), ent.shape[0], most,
+                                          block_tables.data_ptr(), block_tables.shape[1], page,
+                                          _f32(pool), _st(pool)), "pool_blocks")
+    return q_out
+
+
 def window_rows_per_wave(HG: int) -> int:
     """Rows of one sequence portion that a wavefront of the matrix-core window attention takes:
     its 16 (row, head) pairs are RW rows x HS slots for the HG query heads of a key/value head."""
@@ -1047,7 +1252,8 @@ def window_mfma_ok(q, pool, D: int, V: int) -> bool:
 
 def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: int, out, page: int,
                 H: int, G: int, D: int, V: int, units=None, max_keys=None, out_scale: float = 1.0,
-                softcap: float = 0.0, dist=None, gate=None):
+                softcap: float = 0.0, dist=None, gate=None, gate_channels: bool = False,
+                blk=None, every: int = 0):
     """Grouped-query attention over a paged key/value pool with a causal sliding window and a
     softmax sink.
 
@@ -1060,7 +1266,11 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
     softcap c > 0: a score s becomes c * tanh(s / c).  dist = (r1, r2), fp32 [H] each: a key
     d = pos - j positions back loses r1_h * ln(1 + r2_h * d) of its score (after the cap).
     gate: a 2-d view [R, >= H] of the activation type; head h of row r leaves multiplied by
-    sigmoid(gate[r, h]).  Scores, cap, penalty, softmax and gate are fp32.
+    sigmoid(gate[r, h]), or with gate_channels (gate [R, >= H*V]) its channel c by
+    sigmoid(gate[r, h*V + c]).  Scores, cap, penalty, softmax and gate are fp32.
+    blk: a pool of blocks of ``every`` tokens (``conv_rope_norm_store``); beside the window a row sees
+    one key and value for every block that ends before it, (b + 1) * every <= pos - win + 1, in the
+    same softmax (not together with dist).
     units: ``make_units(entries, window_rows_per_wave(H // G))`` on the device; with it bf16
     inputs run on the matrix cores (``window_mfma_ok``)."""
     R = q.shape[0]
@@ -1073,6 +1283,10 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
             j = torch.arange(lo, p + 1)
             tok = bt[int(row_ent[r])][j // page] * page + j % page
             kv = pool[tok].float()
+            if blk is not None:
+                t_ = torch.arange(1, lo // every + 1) * every - 1       # last tokens of the blocks
+                rows = bt[int(row_ent[r])][t_ // page] * blocks_per_page(page, every) + t_ % page // every
+                kv = torch.cat([blk[rows].float(), kv], 0)
             k = kv[:, :G * D].view(-1, G, D).repeat_interleave(HG, 1)       # [n, H, D]
             v = kv[:, G * D:].view(-1, G, V).repeat_interleave(HG, 1)
             s = torch.einsum("hd,nhd->hn", q[r].float().view(H, D), k) * scale
@@ -1085,7 +1299,8 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
             den = e.sum(-1) if sink is None else e.sum(-1) + torch.exp(sink - m)
             o = torch.einsum("hn,nhv->hv", e / den[:, None], v)
             if gate is not None:
-                o = o * torch.sigmoid(gate[r, :H].float())[:, None]
+                o = o * torch.sigmoid(gate[r, :H * V].float().view(H, V) if gate_channels
+                                      else gate[r, :H].float()[:, None])
             out[r] = (o.reshape(H * V) * out_scale).to(out.dtype)
         return out
     _rows2d(q, "q")
@@ -1107,8 +1322,12 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
     ldg = 0
     if gate is not None:
         _rows2d(gate, "gate")
-        assert gate.shape[0] >= R and gate.shape[1] >= H and gate.dtype == q.dtype
+        assert gate.shape[0] >= R and gate.shape[1] >= (H * V if gate_channels else H) and gate.dtype == q.dtype
         ldg = gate.stride(0)
+    if blk is not None:
+        assert every >= 1 and dist is None and blk.is_contiguous() and blk.dtype == pool.dtype
+        assert blk.shape == (pool.shape[0] // page * blocks_per_page(page, every), pool.shape[1])
+    gpc = 1 if gate_channels else 0
     if units is not None and window_mfma_ok(q, pool, D, V):
         assert units.dtype == torch.int32 and units.is_contiguous() and units.shape[1] == 2
         U = units.shape[0]
@@ -1116,7 +1335,8 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
         blocks = U * G * (-(-HG // hs))
         splits = 1
         if max_keys is not None and blocks < LATENT_SPLIT_BLOCKS:
-            splits = max(1, min(-(-min(max_keys, win) // 64), LATENT_SPLIT_BLOCKS // blocks, 64))
+            most = min(max_keys, win) + (max(0, max_keys - win) // every if blk is not None else 0)
+            splits = max(1, min(-(-most // 64), LATENT_SPLIT_BLOCKS // blocks, 64))
         part = None
         if splits > 1:
             L = lib()
@@ -1129,14 +1349,15 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
                                            _lib.ptr(sink), scale, win, out.data_ptr(),
                                            out.stride(0), H, G, D, V, page, splits, _lib.ptr(part),
                                            out_scale, softcap, _lib.ptr(r1), _lib.ptr(r2),
-                                           _lib.ptr(gate), ldg, _st(q)), "window_attn_mfma")
+                                           _lib.ptr(gate), ldg, gpc, _lib.ptr(blk), every, _st(q)),
+             "window_attn_mfma")
         return out
     _chk(lib().p2p_sm_window_attn(q.data_ptr(), q.stride(0), pool.data_ptr(),
                                   block_tables.data_ptr(), block_tables.shape[1],
                                   row_ent.data_ptr(), pos.data_ptr(), _lib.ptr(sink), scale, win,
                                   out.data_ptr(), out.stride(0), R, H, G, D, V, page, out_scale,
-                                  softcap, _lib.ptr(r1), _lib.ptr(r2), _lib.ptr(gate), ldg,
-                                  _f32(q), _st(q)), "window_attn")
+                                  softcap, _lib.ptr(r1), _lib.ptr(r2), _lib.ptr(gate), ldg, gpc,
+                                  _lib.ptr(blk), every, _f32(q), _st(q)), "window_attn")
     return out
 
 
@@ -1188,6 +1409,33 @@ def hgrn2_scan(proj, lower, fb, normw, state, ent, ent_host, out, H: int, D: int
                                  normw.data_ptr(), state.data_ptr(), ent.data_ptr(), ent.shape[0],
                                  out.data_ptr(), out.stride(0), H, D, V, eps, out_scale,
                                  _f32(proj), _st(proj)), "hgrn2_scan")
+    return out
+
+
+def lightning_scan(proj, decay, state, ent, ent_host, out, H: int, D: int, V: int):
+    """Lightning attention.  proj = [q (H*D) | k (H*D) | v (H*V) | ..] raw projections of the step's
+    rows, each through silu; per head S <- decay_h S + k v^T, o = S^T q (o from the updated S).
+    decay fp32 [H]; state fp32 [slots, H, D, V]; out fp32 [R, H*V] (the norm spans the heads and
+    comes after: ``norm_gate``)."""
+    n = H * D
+    if not proj.is_cuda:
+        for row0, cnt, start, slot in ent_host:
+            S = state[slot] if start > 0 else torch.zeros_like(state[slot])
+            for t in range(row0, row0 + cnt):
+                u = torch.nn.functional.silu(proj[t, :2 * n + H * V].float())
+                q, k, v = u[:n].view(H, D), u[n:2 * n].view(H, D), u[2 * n:].view(H, V)
+                S = decay[:, None, None] * S + k[:, :, None] * v[:, None, :]
+                out[t] = torch.einsum("hdv,hd->hv", S, q).reshape(H * V)
+            state[slot] = S
+        return out
+    _rows2d(proj, "proj")
+    _rows2d(out, "out")
+    assert proj.shape[1] >= 2 * n + H * V and out.shape[1] == H * V and out.dtype == torch.float32
+    _vec(decay, H, "decay")
+    _scan_state_ok(state, H, D, V, ent)
+    _chk(lib().p2p_sm_lightning_scan(proj.data_ptr(), proj.stride(0), decay.data_ptr(),
+                                     state.data_ptr(), ent.data_ptr(), ent.shape[0], out.data_ptr(),
+                                     out.stride(0), H, D, V, _f32(proj), _st(proj)), "lightning_scan")
     return out
 
 
