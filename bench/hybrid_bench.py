@@ -1,15 +1,16 @@
-"""Prefill and decode throughput of hybrid models (Regesun, Rotutar, Futetar, Tarunex) at layer sizes that
+"""Prefill and decode throughput of hybrid models (Regesun, Rotutar, Futetar, Tarunex, Rasepel) at layer sizes that
 resemble real models, beside a dense Llama of the same width, depth and parameter count on
 the same engine entry point (``generate``).  Random weights, random tokens.
 
-    python bench.py --hybrid [--hybrid-design regesun|rotutar|futetar|tarunex|both] [--hybrid-sizes 1024,2048]
+    python bench.py --hybrid [--hybrid-design regesun|rotutar|futetar|tarunex|rasepel|both] [--hybrid-sizes 1024,2048]
                     [--steps K] [--warmup W]
 
 ``--hybrid-design rotutar`` runs Rotutar beside Regesun (the closest model: same engine, same
 width and depth) instead of the Llama; ``futetar`` runs Futetar beside Rotutar (gated scans,
 grouped-query attention and routed experts in both); ``tarunex`` runs Tarunex beside Futetar
 (parallel layers, grouped-query attention and routed experts with a shared expert in both; 16
-layer runs each).
+layer runs each); ``rasepel`` runs Rasepel beside Regesun (the same skeleton: three layers of linear
+recurrences for every windowed attention with a clamped dense feed-forward).
 
 One JSON line per (size, model): prefill tokens/s of one long prompt (``prompt`` tokens),
 decode tokens/s of ``batch`` sequences.  These lines are not the headline metric.
@@ -110,6 +111,28 @@ def tarunex_config(width: int):
          "loop": {"start": 2, "stop": 8, "times": 2}, "layers": layers}, name="tarunex-w%d" % width)
 
 
+def rasepel_config(width: int):
+    """A Rasepel stack at a given width: blocks of mamba / lightning / mamba / attention+dense ff, 16
+    states per mamba channel, 128-wide heads, a window of 1024 tokens with blocks of 16 before it."""
+    from p2p_llm_chat_go_amd.models.hybrid import HybridConfig
+
+    hd = 128
+    nh = width // hd
+    mb = {"type": "mamba1", "mixer": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4},
+          "mlp": None}
+    lg = {"type": "lightning", "mixer": {"heads": nh, "dim": hd, "vdim": hd,
+                                         "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * i / nh) for i in range(nh)]},
+          "mlp": None}
+    at = {"type": "attention",
+          "mixer": {"heads": nh, "kv_heads": max(1, nh // 4), "dim": hd, "vdim": hd, "conv": 4,
+                    "mask": {"size": 1024, "pool": 16}, "rot": {"base": 500000.0, "dims": 64},
+                    "scale": hd ** -0.5},
+          "mlp": {"kind": "dense", "ff": 4 * width, "limit": 7.0}}
+    return HybridConfig.from_dict(
+        {"architecture": "Rasepel", "width": width, "vocab": 32000, "norm": {"eps": 1e-5},
+         "embedding": {"scale": 1.0}, "layers": [mb, lg, mb, at] * 4}, name="rasepel-w%d" % width)
+
+
 def n_params(cfg) -> int:
     from p2p_llm_chat_go_amd.models.hybrid import tensor_shapes
 
@@ -179,6 +202,7 @@ def run(a):
         todo = {"regesun": lambda: (hcfg, lcfg), "rotutar": lambda: (rotutar_config(width), hcfg),
                 "futetar": lambda: (futetar_config(width), rotutar_config(width)),
                 "tarunex": lambda: (tarunex_config(width), futetar_config(width)),
+                "rasepel": lambda: (rasepel_config(width), hcfg),
                 "both": lambda: (rotutar_config(width), hcfg, lcfg)}[design]()
         for cfg in todo:
             if getattr(a, "hybrid_only", None) and a.hybrid_only not in cfg.name:

@@ -57,8 +57,9 @@ struct ScanArgs {
   // matrix memory: proj = [q (H*D) | k (H*D) | v (H*V) | gate (H*V) | ...] and the
   // coefficients (a_t, b_t, exp(-m_t)) fp32 [rows, H, 3]
   const float* coef;
-  // lightning: proj = [q (H*D) | k (H*D) | v (H*V) | ...], decay fp32 [H]; out is fp32
-  const float* decay;
+  // lightning: proj = [q (H*D) | k (H*D) | v (H*V) | ...]; pw fp32 [H, ldw], the powers of every
+  // head's decay (column 1 is the decay); out is fp32
+  const float* pw; int ldw;
   int VS;   // value columns of the state: V, or V + 1 with the normaliser
   // common
   const float* normw; float* state; const int* ent; void* out; int ldo;
@@ -158,7 +159,7 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
           float kr = ldf(proj, row * a.ldp + H * D + h * D + i);
           vq = qr * sigmoidf_(qr);
           vk = kr * sigmoidf_(kr);
-          vg = a.decay[h];
+          vg = a.pw[(size_t)h * a.ldw + 1];
         } else {
           float qr = ldf(proj, row * a.ldp + h * D + i);
           vq = qr * sigmoidf_(qr);
@@ -557,11 +558,11 @@ static int launch_chunked(ScanArgs a, const int* vent, int NV, const int* cent, 
 extern "C" {
 
 // portions in one pass; out fp32 [R, H*V] (no norm)
-int p2p_sm_lightning_scan(const void* proj, int ldp, const float* decay, float* state,
+int p2p_sm_lightning_scan(const void* proj, int ldp, const float* pw, int ldw, float* state,
                           const int* ent, int E, float* out, int ldo, int H, int D, int V, int f32,
                           hipStream_t st) {
   ScanArgs a = {};
-  a.proj = proj; a.ldp = ldp; a.decay = decay;
+  a.proj = proj; a.ldp = ldp; a.pw = pw; a.ldw = ldw;
   a.state = state; a.ent = ent; a.out = out; a.ldo = ldo;
   a.H = H; a.G = H; a.D = D; a.V = V;
   return launch_scan<3>(a, E, f32, st);

@@ -130,6 +130,12 @@ def _hybrid_presets() -> dict:
           "mixer": {"heads": 4, "dim": 32, "rot_dim": 16, "vdim": 32, "kv_rank": 64, "q_rank": 96,
                     "rot": {"base": 10000.0, "dims": 16}, "scale": 48 ** -0.5}}
     tmoe = {"kind": "moe", "expert": {"ff": 128}, "shared": {"ff": 256}, "router": {"experts": 8, "top": 2}}
+    m1 = {"type": "mamba1", "mixer": {"inner": 384, "state": 16, "dt_rank": 16, "conv": 4}}
+    li = {"type": "lightning", "mixer": {"heads": 4, "dim": 48, "vdim": 64, "decay": [0.75, 0.9, 0.97, 0.995]}}
+    ca = {"type": "attention",
+          "mixer": {"heads": 8, "kv_heads": 2, "dim": 32, "vdim": 32, "conv": 3, "scale": 32 ** -0.5,
+                    "mask": {"size": 128, "pool": 8}, "rot": {"base": 10000.0, "dims": 32}}}
+    clamp = {"kind": "dense", "ff": 512, "limit": 7.0}
     return {"tiny-regesun": HybridConfig.from_dict(
         {"architecture": "Regesun", "width": 256, "vocab": 512, "max_positions": 4096,
          "norm": {"eps": 1e-5}, "layers": [gd, mb, la, mb, gd, la], "eos_token_id": [2]},
@@ -148,12 +154,17 @@ def _hybrid_presets() -> dict:
          "embedding": {"scale": 16.0}, "logit_scale": 0.5, "logit_softcap": 25.0,
          "loop": {"start": 1, "stop": 3, "times": 2},
          "layers": [dict(ba, mlp=tmoe), dict(rl, mlp=tmoe), dict(ba, mlp=tmoe), dict(rl, mlp=None)],
-         "eos_token_id": [2]}, name="tiny-tarunex")}
+         "eos_token_id": [2]}, name="tiny-tarunex"),
+        "tiny-rasepel": HybridConfig.from_dict(
+        {"architecture": "Rasepel", "width": 256, "vocab": 512, "norm": {"eps": 1e-5},
+         "embedding": {"scale": 4.0},
+         "layers": [dict(m1, mlp=clamp), dict(ca, mlp=clamp), dict(li, mlp=clamp), dict(ca, mlp=None), m1],
+         "eos_token_id": [2]}, name="tiny-rasepel")}
 
 
 def get_config(name: str):
     key = ALIASES.get(name, name)
-    if key not in PRESETS and key.endswith(("regesun", "rotutar", "futetar", "tarunex")):
+    if key not in PRESETS and key.endswith(("regesun", "rotutar", "futetar", "tarunex", "rasepel")):
         hp = _hybrid_presets()
         if key in hp:
             return hp[key]

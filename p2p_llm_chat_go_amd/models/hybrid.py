@@ -517,7 +517,7 @@ class Lightning(Mixer):
         self._dims()
         # one projection for everything that reads the layer input: q | k | v | gate
         self.w_in = torch.cat([get(k) for k in ("q", "k", "v", "g")], 0).to(dev, dtype).contiguous()
-        self.lam = torch.tensor(self.decay, dtype=torch.float32, device=dev)
+        self.powers = sm.decay_powers(self.decay, dev)
         self.normw = _vec(get("norm"), dev)
         self.wo = get("o").to(dev, dtype).contiguous()
 
@@ -527,7 +527,7 @@ class Lightning(Mixer):
     def mix(self, proj, b, cache, layer, out, out_scale=1.0):
         H, D, V = self.H, self.D, self.V
         o = torch.empty(b.R, H * V, device=proj.device, dtype=torch.float32)
-        sm.lightning_scan(proj, self.lam, cache.state[layer]["S"], b.ent, b.ent_host, o, H, D, V)
+        sm.lightning_scan(proj, self.powers, cache.state[layer]["S"], b.ent, b.ent_host, o, H, D, V)
         g0 = 2 * H * D + H * V
         sm.norm_gate(o, self.normw, proj[:, g0:g0 + H * V], self.eps, out)
         if out_scale != 1.0:

@@ -66,8 +66,10 @@ _SIGS = {
     "p2p_sm_selective_step": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
                               c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                               c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
-    "p2p_sm_lightning_scan": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
+    "p2p_sm_lightning_scan": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int,
                               c_int, c_int, c_int, c_int, c_void_p],
+    "p2p_sm_lightning_chunked": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                                 c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
@@ -1412,12 +1414,23 @@ def hgrn2_scan(proj, lower, fb, normw, state, ent, ent_host, out, H: int, D: int
     return out
 
 
-def lightning_scan(proj, decay, state, ent, ent_host, out, H: int, D: int, V: int):
+LIGHT_CHUNK = 64      # tokens of a chunk of the matrix-instruction kernels
+LIGHT_MIN = int(os.environ.get("P2P_LIGHT_MIN", "32"))   # portions from here on run in chunks
+
+
+def decay_powers(decay, device) -> torch.Tensor:
+    """fp32 [H, LIGHT_CHUNK + 1]: decay_h^0 .. decay_h^LIGHT_CHUNK, formed in float64."""
+    d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
+    return torch.pow(d[:, None], torch.arange(LIGHT_CHUNK + 1, dtype=torch.float64)).float().contiguous().to(device)
+
+
+def lightning_scan(proj, powers, state, ent, ent_host, out, H: int, D: int, V: int):
     """Lightning attention.  proj = [q (H*D) | k (H*D) | v (H*V) | ..] raw projections of the step's
     rows, each through silu; per head S <- decay_h S + k v^T, o = S^T q (o from the updated S).
-    decay fp32 [H]; state fp32 [slots, H, D, V]; out fp32 [R, H*V] (the norm spans the heads and
+    powers: ``decay_powers`` of the heads' decays; state fp32 [slots, H, D, V]; out fp32 [R, H*V] (the norm spans the heads and
     comes after: ``norm_gate``)."""
     n = H * D
+    decay = powers[:, 1]
     if not proj.is_cuda:
         for row0, cnt, start, slot in ent_host:
             S = state[slot] if start > 0 else torch.zeros_like(state[slot])
@@ -1431,10 +1444,19 @@ def lightning_scan(proj, decay, state, ent, ent_host, out, H: int, D: int, V: in
     _rows2d(proj, "proj")
     _rows2d(out, "out")
     assert proj.shape[1] >= 2 * n + H * V and out.shape[1] == H * V and out.dtype == torch.float32
-    _vec(decay, H, "decay")
+    assert powers.dtype == torch.float32 and powers.is_contiguous() and powers.shape == (H, LIGHT_CHUNK + 1)
     _scan_state_ok(state, H, D, V, ent)
-    _chk(lib().p2p_sm_lightning_scan(proj.data_ptr(), proj.stride(0), decay.data_ptr(),
-                                     state.data_ptr(), ent.data_ptr(), ent.shape[0], out.data_ptr(),
+    if max(e[1] for e in ent_host) >= LIGHT_MIN:
+        vent, cent = (t_.to(proj.device) for t_ in scan_chunks(ent_host, LIGHT_CHUNK))
+        NV = vent.shape[0]
+        cs = torch.empty(NV, H, D, V, device=proj.device, dtype=torch.float32)
+        _chk(lib().p2p_sm_lightning_chunked(proj.data_ptr(), proj.stride(0), powers.data_ptr(),
+                                            state.data_ptr(), vent.data_ptr(), NV, cent.data_ptr(),
+                                            ent.shape[0], cs.data_ptr(), out.data_ptr(), out.stride(0),
+                                            H, D, V, _f32(proj), _st(proj)), "lightning_chunked")
+        return out
+    _chk(lib().p2p_sm_lightning_scan(proj.data_ptr(), proj.stride(0), powers.data_ptr(),
+                                     powers.stride(0), state.data_ptr(), ent.data_ptr(), ent.shape[0], out.data_ptr(),
                                      out.stride(0), H, D, V, _f32(proj), _st(proj)), "lightning_scan")
     return out
 
