@@ -104,16 +104,121 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D,
   }
 }
 
-// blocks that the step's portions of more than one token complete; one workgroup per (block,
+// The same for prompts, RT consecutive rows per workgroup: the angles of a row are formed once for
+// all heads (sincos in LDS), every wavefront takes heads 4 apart and walks the rows of one with
+// the taps and the window of its channels in registers.  Head sizes up to 256, KT taps.  It
+// neither moves tails nor forms blocks.
+#define RT 8
+template <typename T, int KT>
+__global__ void __launch_bounds__(256)
+conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int D, int V,
+                      const float* __restrict__ cw, const float* __restrict__ tail,
+                      const int* __restrict__ ent, const int* __restrict__ row_ent,
+                      const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
+                      float eps, const int* __restrict__ pos, const int* __restrict__ cache_rows,
+                      T* __restrict__ pool, T* __restrict__ q_out, int ldq, int R, int LDS) {
+  constexpr int NM = 4;               // channels of a lane at most
+  extern __shared__ float smem[];     // [RT][nrot][2] cos | sin, then a head per wavefront
+  const int r0 = blockIdx.x * RT, nr = min(RT, R - r0);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float* s = smem + RT * nrot * 2 + wave * LDS;
+  for (int idx = threadIdx.x; idx < nr * nrot; idx += 256) {
+    float sn, cs;
+    sincosf((float)pos[r0 + idx / nrot] * inv_freq[idx % nrot], &sn, &cs);
+    smem[2 * idx] = cs;
+    smem[2 * idx + 1] = sn;
+  }
+  __syncthreads();
+  const int C = (H + G) * D + G * V, W = G * (D + V);
+  for (int hh = wave; hh < H + 2 * G; hh += 4) {
+    const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
+    const int hd = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
+    const int n = kind == 2 ? V : D;
+    const int c0 = kind == 0 ? hd * D : kind == 1 ? (H + hd) * D : (H + G) * D + hd * V;
+    const float tq = kind == 0 && temp ? temp[hd] : 1.0f;
+    float w[NM][KT], u[NM][KT - 1];
+#pragma unroll
+    for (int m = 0; m < NM; m++) {
+      const int c = c0 + min(lane + 64 * m, n - 1);
+      if (64 * m < n) {
+#pragma unroll
+        for (int kk = 0; kk < KT; kk++) w[m][kk] = cw[(size_t)c * KT + kk];
+#pragma unroll
+        for (int kk = 0; kk < KT - 1; kk++)
+          u[m][kk] = ldf(proj, (size_t)max(r0 - (KT - 1) + kk, 0) * ldp + c);
+      }
+    }
+    float nx[NM];
+#pragma unroll
+    for (int m = 0; m < NM; m++)
+      nx[m] = 64 * m < n ? ldf(proj, (size_t)r0 * ldp + c0 + min(lane + 64 * m, n - 1)) : 0.0f;
+    for (int i = 0; i < nr; i++) {
+      const int r = r0 + i;
+      const Entry en = load_entry(ent, row_ent[r]);
+      const int t = r - en.row0;
+      float cur[NM];
+#pragma unroll
+      for (int m = 0; m < NM; m++) cur[m] = nx[m];
+      if (i + 1 < nr) {
+#pragma unroll
+        for (int m = 0; m < NM; m++)
+          if (64 * m < n) nx[m] = ldf(proj, (size_t)(r + 1) * ldp + c0 + min(lane + 64 * m, n - 1));
+      }
+#pragma unroll
+      for (int m = 0; m < NM; m++) {
+        if (64 * m >= n) break;
+        const int ch = lane + 64 * m, c = c0 + min(ch, n - 1);
+        float acc = 0.0f;
+#pragma unroll
+        for (int kk = 0; kk < KT - 1; kk++) {
+          const int q = t - (KT - 1) + kk;
+          float v = u[m][kk];
+          if (q < 0) v = en.start > 0 ? tail[((size_t)en.slot * (KT - 1) + (KT - 1 + q)) * C + c] : 0.0f;
+          acc += w[m][kk] * v;
+        }
+        acc += w[m][KT - 1] * cur[m];
+#pragma unroll
+        for (int kk = 0; kk + 1 < KT - 1; kk++) u[m][kk] = u[m][kk + 1];
+        u[m][KT - 2] = cur[m];
+        if (ch < n) s[ch] = acc;
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      T* crow = pool + (size_t)cache_rows[r] * W;
+      T* dst = kind == 0 ? q_out + (size_t)r * ldq + hd * D : kind == 1 ? crow + hd * D
+                                                                        : crow + G * D + hd * V;
+      float rs = 1.0f;
+      if (kind < 2) {
+        float ss = 0.0f;
+        for (int j = lane; j < nrot; j += 64) {
+          const float a = s[j], b = s[j + nrot];
+          const float cs = smem[2 * (i * nrot + j)], sn = smem[2 * (i * nrot + j) + 1];
+          const float x = a * cs - b * sn, y = b * cs + a * sn;
+          s[j] = x;
+          s[j + nrot] = y;
+          ss += x * x + y * y;
+        }
+        for (int k = 2 * nrot + lane; k < n; k += 64) ss += s[k] * s[k];
+        ss = wave_sum(ss);
+        rs = 1.0f / sqrtf(ss / (float)n + eps) * tq;
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      for (int k = lane; k < n; k += 64) stf(dst, k, s[k] * rs);
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");   // before the next row overwrites s
+    }
+  }
+}
+
+// blocks that the step's portions of at least min_n tokens complete; one workgroup per (block,
 // entry), grid.x covers the entry with most of them
 template <typename T>
 __global__ void __launch_bounds__(256)
 pool_blocks_k(const T* __restrict__ pool, int W, T* __restrict__ blk, int P,
-              const int* __restrict__ ent, const int* __restrict__ bt, int max_pages, int page) {
+              const int* __restrict__ ent, const int* __restrict__ bt, int max_pages, int page,
+              int min_n) {
   const int e = blockIdx.y;
   const Entry en = load_entry(ent, e);
   const int last = (en.start / P + blockIdx.x) * P + P - 1;
-  if (en.n < 2 || last >= en.start + en.n) return;
+  if (en.n < min_n || last >= en.start + en.n) return;
   const int* pages = bt + (size_t)e * max_pages;
   T* brow = blk + ((size_t)pages[last / page] * ((page + P - 1) / P) + (last % page) / P) * W;
   for (int c = threadIdx.x; c < W; c += blockDim.x) {
@@ -134,19 +239,35 @@ pool_blocks_k(const T* __restrict__ pool, int W, T* __restrict__ blk, int P,
 
 extern "C" {
 
+// rows: several rows per workgroup (3 or 4 taps, head sizes up to 256); the tails and blocks of
+// every portion, also of single tokens, are then left to other kernels
 int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, int V,
                                 const float* cw, int K, float* tail, const int* ent,
                                 const int* row_ent, const float* inv_freq, int nrot,
                                 const float* temp, float eps, const int* pos,
                                 const int* cache_rows, void* pool, void* q_out, int ldq, void* blk,
-                                int P, const int* bt, int max_pages, int page, int R, int f32,
-                                hipStream_t st) {
+                                int P, const int* bt, int max_pages, int page, int R, int rows,
+                                int f32, hipStream_t st) {
   if (R <= 0) return 0;
   if (H < 1 || G < 1 || D < 1 || V < 1 || K < 1 || nrot < 0 || 2 * nrot > D || page < 1 ||
       (blk && P < 1))
     return (int)hipErrorInvalidValue;
   const int LDS = D > V ? D : V;
   if ((size_t)4 * LDS * 4 > 64 * 1024) return (int)hipErrorInvalidValue;
+  const size_t shm = ((size_t)RT * nrot * 2 + 4 * LDS) * 4;
+  if (rows) {
+    if ((K != 4 && K != 3) || LDS > 256 || shm > 64 * 1024) return (int)hipErrorInvalidValue;
+    dim3 gr((R + RT - 1) / RT);
+#define CRN(KT)                                                                                   \
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL((conv_rope_norm_rows_k<T, KT>), gr, dim3(256), shm, st,   \
+                                         (const T*)proj, ldp, H, G, D, V, cw, tail, ent, row_ent, \
+                                         inv_freq, nrot, temp, eps, pos, cache_rows, (T*)pool,    \
+                                         (T*)q_out, ldq, R, LDS))
+    if (K == 4) CRN(4);
+    else CRN(3);
+#undef CRN
+    return (int)hipGetLastError();
+  }
   dim3 grid(R, (H + 2 * G + 3) / 4);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(conv_rope_norm_store_k<T>, grid, dim3(256),
                                          (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, D, V,
@@ -158,13 +279,13 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, 
 
 // max_blocks: the most blocks a portion of the step completes
 int p2p_sm_pool_blocks(const void* pool, int W, void* blk, int P, const int* ent, int E,
-                       int max_blocks, const int* bt, int max_pages, int page, int f32,
+                       int max_blocks, const int* bt, int max_pages, int page, int min_n, int f32,
                        hipStream_t st) {
   if (E <= 0 || max_blocks <= 0) return 0;
   if (P < 1 || W < 1 || page < 1) return (int)hipErrorInvalidValue;
   dim3 grid(max_blocks, E);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(pool_blocks_k<T>, grid, dim3(256), 0, st, (const T*)pool,
-                                         W, (T*)blk, P, ent, bt, max_pages, page));
+                                         W, (T*)blk, P, ent, bt, max_pages, page, min_n));
   return (int)hipGetLastError();
 }
 

@@ -42,6 +42,48 @@ __global__ void mamba_conv_k(const T* __restrict__ zx, int ldz, int xoff,
   }
 }
 
+// The same for prompts: a thread walks CR consecutive rows of its channel, so the taps are read once
+// and every raw input once (its window stays in registers); all of its loads go out together.
+// Rows whose window reaches before their portion take it from the tail, row by row.
+#define CR 8
+template <typename T, typename TO, int KT>
+__global__ void mamba_conv_rows_k(const T* __restrict__ zx, int ldz, int xoff,
+                                  const float* __restrict__ cw, const float* __restrict__ cb,
+                                  const float* __restrict__ tail, const int* __restrict__ ent,
+                                  const int* __restrict__ row_ent, TO* __restrict__ out, int ldo,
+                                  int R, int C) {
+  const int c = blockIdx.x * blockDim.x + threadIdx.x, r0 = blockIdx.y * CR;
+  if (c >= C) return;
+  float w[KT], u[CR + KT - 1];
+#pragma unroll
+  for (int kk = 0; kk < KT; kk++) w[kk] = cw[(size_t)c * KT + kk];
+#pragma unroll
+  for (int i = 0; i < CR + KT - 1; i++)
+    u[i] = ldf(zx, (size_t)min(max(r0 + i - (KT - 1), 0), R - 1) * ldz + xoff + c);
+  const float b = cb[c];
+#pragma unroll
+  for (int i = 0; i < CR; i++) {
+    const int r = r0 + i;
+    if (r >= R) break;
+    const Entry en = load_entry(ent, row_ent[r]);
+    const int t = r - en.row0;
+    float acc = b;
+    if (t >= KT - 1) {
+#pragma unroll
+      for (int kk = 0; kk < KT; kk++) acc += w[kk] * u[i + kk];
+    } else {
+#pragma unroll
+      for (int kk = 0; kk < KT; kk++) {
+        const int q = t - (KT - 1) + kk;
+        float v = u[i + kk];
+        if (q < 0) v = en.start > 0 ? tail[((size_t)en.slot * (KT - 1) + (KT - 1 + q)) * C + c] : 0.0f;
+        acc += w[kk] * v;
+      }
+    }
+    stf(out, (size_t)r * ldo + c, acc * sigmoidf_(acc));
+  }
+}
+
 // One thread owns NSUB consecutive state rows of one value column: thread (p, ns) holds
 // S[ns * NSUB + q][p].  Per token it updates them and leaves its share of y = S^T C in LDS;
 // the shares are added, D x and the gate applied, once per staged chunk of tokens.
@@ -214,6 +256,20 @@ int p2p_sm_mamba_conv(const void* zx, int ldz, int xoff, const float* cw, const 
   if (R <= 0) return 0;
   if (K < 1) return (int)hipErrorInvalidValue;
   dim3 g((C + 255) / 256, R), b(256);
+  // portions of one token roll their tails in the other kernel, which a step of many rows
+  // without the request does not need
+  if (!roll && R >= 64 && (K == 4 || K == 3)) {
+    g.y = (R + CR - 1) / CR;
+#define CONV_ROWS(TO, KT)                                                                         \
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL((mamba_conv_rows_k<T, TO, KT>), g, b, 0, st, (const T*)zx, \
+                                         ldz, xoff, cw, cb, tail, ent, row_ent, (TO*)out, ldo, R, C))
+    if (out_f32 && K == 4) CONV_ROWS(float, 4);
+    else if (out_f32) CONV_ROWS(float, 3);
+    else if (K == 4) CONV_ROWS(T, 4);
+    else CONV_ROWS(T, 3);
+#undef CONV_ROWS
+    return (int)hipGetLastError();
+  }
   if (out_f32)
     SM_DISPATCH_T(f32, hipLaunchKernelGGL((mamba_conv_k<T, float>), g, b, 0, st, (const T*)zx, ldz,
                                            xoff, cw, cb, tail, ent, row_ent, (float*)out, ldo, C,

@@ -397,7 +397,7 @@ __global__ void gate_norm_add_k(float* __restrict__ x, const T* __restrict__ y, 
 
 // out = x / sqrt(mean(x^2) + eps) * w * sigmoid(g): the norm of a whole fp32 row (all heads of a
 // recurrence together) with a gate per channel, on the way into an output projection
-template <typename T>
+template <typename T, int NR>   // NR: values a thread keeps (rows of up to 256 * NR numbers are read once)
 __global__ void norm_gate_k(const float* __restrict__ x, int ldx, const float* __restrict__ w,
                             const T* __restrict__ g, int ldg, T* __restrict__ out, int ldo, int n,
                             float eps) {
@@ -406,25 +406,25 @@ __global__ void norm_gate_k(const float* __restrict__ x, int ldx, const float* _
   const float* xr = x + (size_t)r * ldx;
   const T* gr = g + (size_t)r * ldg;
   T* o = out + (size_t)r * ldo;
-  if (n <= NV * (int)blockDim.x) {
-    float v[NV], m[NV];
+  if (n <= NR * (int)blockDim.x) {
+    float v[NR], m[NR];
     float ss = 0.0f;
 #pragma unroll
-    for (int k = 0; k < NV; k++) {
+    for (int k = 0; k < NR; k++) {
       int i = threadIdx.x + k * blockDim.x;
       int ic = i < n ? i : 0;
       v[k] = xr[ic];
       m[k] = w[ic] * sigmoidf_(ldf(gr, ic));
     }
 #pragma unroll
-    for (int k = 0; k < NV; k++) {
+    for (int k = 0; k < NR; k++) {
       if (threadIdx.x + k * blockDim.x >= (unsigned)n) v[k] = 0.0f;
       ss += v[k] * v[k];
     }
     ss = block_sum(ss, red);
     float rs = 1.0f / sqrtf(ss / (float)n + eps);
 #pragma unroll
-    for (int k = 0; k < NV; k++) {
+    for (int k = 0; k < NR; k++) {
       int i = threadIdx.x + k * blockDim.x;
       if (i < n) stf(o, i, v[k] * rs * m[k]);
     }
@@ -443,8 +443,13 @@ extern "C" {
 int p2p_sm_norm_gate(const float* x, int ldx, const float* w, const void* g, int ldg, void* out,
                      int ldo, int R, int n, float eps, int f32, hipStream_t st) {
   if (R <= 0 || n <= 0) return 0;
-  SM_DISPATCH_T(f32, hipLaunchKernelGGL(norm_gate_k<T>, dim3(R), dim3(256), 0, st, x, ldx, w,
-                                         (const T*)g, ldg, (T*)out, ldo, n, eps));
+#define NG(NR)                                                                                   \
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL((norm_gate_k<T, NR>), dim3(R), dim3(256), 0, st, x, ldx, w, \
+                                         (const T*)g, ldg, (T*)out, ldo, n, eps))
+  if (n <= 256 * 4) NG(4);
+  else if (n <= 256 * 8) NG(8);
+  else NG(16);
+#undef NG
   return (int)hipGetLastError();
 }
 

@@ -73,9 +73,9 @@ _SIGS = {
     "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
-                                    c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+                                    c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_pool_blocks": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int,
-                           c_int, c_int, c_void_p],
+                           c_int, c_int, c_int, c_void_p],
     "p2p_sm_mamba_scan": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
                           c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int,
                           c_int, c_int, c_int, c_int, c_void_p],
@@ -593,8 +593,8 @@ def mamba_conv(zx, xoff: int, cw, cb, tail, ent, ent_host, row_ent, out, roll: b
     """Causal per-channel convolution + bias + silu over channels [xoff, xoff + C) of zx.
     cw fp32 [C, K] (column K-1 multiplies the newest input), tail fp32 [slots, K-1, C] the raw inputs
     before each slot's next token; out [R, C] fp32 or activation typed.  roll: the tails move
-    forward as well (in the same kernel for portions of one token, ``conv_tail_roll`` for the
-    others); without it they are only read (``mamba_scan`` / ``conv_tail_roll`` follow)."""
+    forward as well (in the same kernel when every portion is one token, else by
+    ``conv_tail_roll``); without it they are only read (``mamba_scan`` / ``conv_tail_roll`` follow)."""
     R, C = out.shape
     K = cw.shape[1]
     if not zx.is_cuda:
@@ -616,12 +616,13 @@ def mamba_conv(zx, xoff: int, cw, cb, tail, ent, ent_host, row_ent, out, roll: b
     _vec(cb, C, "cb")
     assert tail.dtype == torch.float32 and tail.is_contiguous() and tail.shape[1:] == (K - 1, C)
     assert xoff + C <= zx.shape[1] and row_ent.dtype == torch.int32
+    fused = roll and all(e[1] == 1 for e in ent_host)
     _chk(lib().p2p_sm_mamba_conv(zx.data_ptr(), zx.stride(0), xoff, cw.data_ptr(), cb.data_ptr(),
                                  tail.data_ptr(), ent.data_ptr(), row_ent.data_ptr(),
                                  out.data_ptr(), out.stride(0), _f32(out), R, C, K,
-                                 1 if roll else 0, _f32(zx), _st(zx)), "mamba_conv")
-    if roll:
-        conv_tail_roll(zx, xoff, tail, ent, ent_host, C, skip_single=True)
+                                 1 if fused else 0, _f32(zx), _st(zx)), "mamba_conv")
+    if roll and not fused:
+        conv_tail_roll(zx, xoff, tail, ent, ent_host, C)
     return out
 
 
@@ -1220,20 +1221,24 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
         assert blk.shape == (pool.shape[0] // page * sb, pool.shape[1])
     if 4 * max(D, V) * 4 > 64 * 1024:
         raise ValueError("conv_rope_norm_store: head sizes %d / %d" % (D, V))
+    # steps with prompts: several rows per workgroup, then tails and blocks of all portions; else
+    # single tokens move their tails and form their blocks in the first kernel
+    rows = R >= 64 and K in (3, 4) and max(D, V) <= 256 and any(e[1] > 1 for e in ent_host)
     _chk(lib().p2p_sm_conv_rope_norm_store(
         proj.data_ptr(), proj.stride(0), H, G, D, V, cw.data_ptr(), K, tail.data_ptr(),
         ent.data_ptr(), row_ent.data_ptr(), inv_freq.data_ptr(), nrot, _lib.ptr(temp), eps,
         pos.data_ptr(), cache_rows.data_ptr(), pool.data_ptr(), q_out.data_ptr(), q_out.stride(0),
-        _lib.ptr(blk), every, block_tables.data_ptr(), block_tables.shape[1], page, R, _f32(proj),
-        _st(proj)), "conv_rope_norm_store")
-    conv_tail_roll(proj, 0, tail, ent, ent_host, C, skip_single=True)
+        _lib.ptr(blk), every, block_tables.data_ptr(), block_tables.shape[1], page, R,
+        1 if rows else 0, _f32(proj), _st(proj)), "conv_rope_norm_store")
+    conv_tail_roll(proj, 0, tail, ent, ent_host, C, skip_single=not rows)
     if blk is not None:
-        most = max([(e[2] + e[1]) // every - e[2] // every for e in ent_host if e[1] > 1] or [0])
+        least = 1 if rows else 2
+        most = max([(e[2] + e[1]) // every - e[2] // every for e in ent_host if e[1] >= least] or [0])
         if most:
             _chk(lib().p2p_sm_pool_blocks(pool.data_ptr(), pool.shape[1], blk.data_ptr(), every,
                                           ent.data_ptr(), ent.shape[0], most,
                                           block_tables.data_ptr(), block_tables.shape[1], page,
-                                          _f32(pool), _st(pool)), "pool_blocks")
+                                          least, _f32(pool), _st(pool)), "pool_blocks")
     return q_out
 
 
