@@ -104,9 +104,9 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D,
   }
 }
 
-// The same for prompts, RT consecutive rows per workgroup: the angles of a row are formed once for
-// all heads (sincos in LDS), every wavefront takes heads 4 apart and walks the rows of one with
-// the taps and the window of its channels in registers.  Head sizes up to 256, KT taps.  It
+// The same for prompts, RT consecutive rows of four heads per workgroup: the angles of the rows are
+// formed once for its heads (sincos in LDS), every wavefront walks the rows of one head with the
+// taps and the window of its channels in registers.  Head sizes up to 256, KT taps.  It
 // neither moves tails nor forms blocks.
 #define RT 8
 template <typename T, int KT>
@@ -130,7 +130,8 @@ conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int D, 
   }
   __syncthreads();
   const int C = (H + G) * D + G * V, W = G * (D + V);
-  for (int hh = wave; hh < H + 2 * G; hh += 4) {
+  const int hh = blockIdx.y * 4 + wave;
+  if (hh < H + 2 * G) {
     const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
     const int hd = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
     const int n = kind == 2 ? V : D;
@@ -257,7 +258,7 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, 
   const size_t shm = ((size_t)RT * nrot * 2 + 4 * LDS) * 4;
   if (rows) {
     if ((K != 4 && K != 3) || LDS > 256 || shm > 64 * 1024) return (int)hipErrorInvalidValue;
-    dim3 gr((R + RT - 1) / RT);
+    dim3 gr((R + RT - 1) / RT, (H + 2 * G + 3) / 4);
 #define CRN(KT)                                                                                   \
   SM_DISPATCH_T(f32, hipLaunchKernelGGL((conv_rope_norm_rows_k<T, KT>), gr, dim3(256), shm, st,   \
                                          (const T*)proj, ldp, H, G, D, V, cw, tail, ent, row_ent, \

@@ -33,6 +33,24 @@ __global__ void ff_act_k(const T* __restrict__ gu, int ld, T* __restrict__ out, 
   stf(out, (size_t)r * ldo + c, g * sigmoidf_(alpha * g) * (u + 1.0f));
 }
 
+// four neighbouring channels per thread (rows and widths that are multiples of 4)
+template <typename T>
+__global__ void ff_act4_k(const T* __restrict__ gu, int ld, T* __restrict__ out, int ldo, int F,
+                          float limit, float alpha) {
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4, r = blockIdx.y;
+  if (c >= F) return;
+  struct alignas(4 * sizeof(T)) V4 { T v[4]; };
+  const V4 gv = *(const V4*)(gu + (size_t)r * ld + c), uv = *(const V4*)(gu + (size_t)r * ld + F + c);
+  V4 o;
+#pragma unroll
+  for (int i = 0; i < 4; i++) {
+    const float g = fminf(ldf(gv.v, i), limit), u = fminf(fmaxf(ldf(uv.v, i), -limit), limit);
+    stf(o.v, i, g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * g)) *
+                    (u + 1.0f));
+  }
+  *(V4*)(out + (size_t)r * ldo + c) = o;
+}
+
 // tanh form of gelu: 0.5 z (1 + tanh(y)), y = sqrt(2/pi) (z + 0.044715 z^3), evaluated as
 // z * sigmoid(2 y), which is the same function (1 + tanh(y) = 2 sigmoid(2 y))
 __device__ __forceinline__ float gelu_tanhf_(float z) {
@@ -119,6 +137,12 @@ int p2p_sm_sigmoid_gate(const void* o, long soh, long sor, const void* gt, int l
 int p2p_sm_ff_act(const void* gu, int ld, void* out, int ldo, int R, int F, float limit,
                   float alpha, int f32, hipStream_t st) {
   if (R <= 0) return 0;
+  const size_t al = f32 ? 16 : 8;
+  if (F % 4 == 0 && ld % 4 == 0 && ldo % 4 == 0 && (size_t)gu % al == 0 && (size_t)out % al == 0) {
+    SM_DISPATCH_T(f32, hipLaunchKernelGGL(ff_act4_k<T>, dim3((F + 1023) / 1024, R), dim3(256), 0, st,
+                                           (const T*)gu, ld, (T*)out, ldo, F, limit, alpha));
+    return (int)hipGetLastError();
+  }
   dim3 g((F + 255) / 256, R), b(256);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(ff_act_k<T>, g, b, 0, st, (const T*)gu, ld, (T*)out, ldo,
                                          F, limit, alpha));

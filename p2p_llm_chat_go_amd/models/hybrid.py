@@ -276,7 +276,7 @@ class StepBatch:
             r0 += n
         parts = [torch.tensor(x, dtype=torch.int32).reshape(-1)
                  for x in (ids, pos, row_ent, rows, ent, outs or [0])] + [bt.reshape(-1)]
-        meta = {"R": r0, "E": len(entries), "ent_host": ent, "n_out": len(outs),
+        meta = {"R": r0, "E": len(entries), "ent_host": sm.Entries(ent), "n_out": len(outs),
                 "max_pos": max(pos), "maxp": maxp, "sizes": [p.numel() for p in parts]}
         return torch.cat(parts), meta
 

@@ -526,6 +526,29 @@ def scan_chunks(ent_host: list, chunk: int):
     return torch.tensor(vent, dtype=torch.int32), torch.tensor(cent, dtype=torch.int32)
 
 
+class Entries(list):
+    """The entries of one step, (first row, rows, first position, slot) each, with what has been
+    derived from them on the device: every layer of the step asks for the same tables."""
+
+    def __init__(self, entries=()):
+        super().__init__(entries)
+        self.tables = {}
+
+
+def chunk_tables(ent_host: list, chunk: int, device):
+    """``scan_chunks`` on the device, in one copy (kept with the step when it is an ``Entries``)."""
+    kept = getattr(ent_host, "tables", None)
+    key = (chunk, str(device))
+    if kept is not None and key in kept:
+        return kept[key]
+    vent, cent = scan_chunks(ent_host, chunk)
+    both = torch.cat([vent, cent]).to(device)
+    out = both[:vent.shape[0]], both[vent.shape[0]:]
+    if kept is not None:
+        kept[key] = out
+    return out
+
+
 def _chunked(ent_host) -> bool:
     return SCAN_CHUNK > 0 and max(e[1] for e in ent_host) >= 2 * SCAN_CHUNK
 
@@ -572,7 +595,7 @@ def gdelta_scan(r, k, v, g, a, lo, w0, ab, normw, state, ent, ent_host, out, H: 
     if D > 256:
         raise ValueError("gdelta_scan: head size %d > 256" % D)
     if _chunked(ent_host):
-        vent, cent = (t_.to(r.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, r.device)
         tmp = torch.empty(3, vent.shape[0], H, D, D, device=r.device, dtype=torch.float32)
         _chk(lib().p2p_sm_gdelta_scan_chunked(
             r.data_ptr(), k.data_ptr(), v.data_ptr(), g.data_ptr(), a.data_ptr(), ld,
@@ -692,7 +715,7 @@ def mamba_scan(conv, zx, xoff: int, dtoff: int, dt_bias, A_log, Dp, state, tail,
         raise ValueError("mamba_scan: state %d / value %d sizes above 256" % (N, P))
     E = ent.shape[0]
     if _chunked(ent_host):
-        vent, cent = (t_.to(zx.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, zx.device)
         NV = vent.shape[0]
         tmp = torch.empty(NV, H, N, P, device=zx.device, dtype=torch.float32)
         decay = torch.empty(NV, H, device=zx.device, dtype=torch.float32)
@@ -765,7 +788,7 @@ def selective_scan(x, xp, rank: int, wdt, dt_bias, A2, Dp, z, state, ent, ent_ho
     vent = cent = tmp = dtsum = None
     NV = 0
     if _chunked(ent_host):
-        vent, cent = (t_.to(y.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, y.device)
         NV = vent.shape[0]
         tmp = torch.empty(NV, N, I, device=y.device, dtype=torch.float32)
         dtsum = torch.empty(NV, I, device=y.device, dtype=torch.float32)
@@ -1402,7 +1425,7 @@ def hgrn2_scan(proj, lower, fb, normw, state, ent, ent_host, out, H: int, D: int
     _vec(normw, V, "normw")
     _scan_state_ok(state, H, D, V, ent)
     if _chunked(ent_host):
-        vent, cent = (t_.to(proj.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, proj.device)
         NV = vent.shape[0]
         cs = torch.empty(NV, H, D, V, device=proj.device, dtype=torch.float32)
         cd = torch.empty(NV, H, D, device=proj.device, dtype=torch.float32)
@@ -1452,7 +1475,7 @@ def lightning_scan(proj, powers, state, ent, ent_host, out, H: int, D: int, V: i
     assert powers.dtype == torch.float32 and powers.is_contiguous() and powers.shape == (H, LIGHT_CHUNK + 1)
     _scan_state_ok(state, H, D, V, ent)
     if max(e[1] for e in ent_host) >= LIGHT_MIN:
-        vent, cent = (t_.to(proj.device) for t_ in scan_chunks(ent_host, LIGHT_CHUNK))
+        vent, cent = chunk_tables(ent_host, LIGHT_CHUNK, proj.device)
         NV = vent.shape[0]
         cs = torch.empty(NV, H, D, V, device=proj.device, dtype=torch.float32)
         _chk(lib().p2p_sm_lightning_chunked(proj.data_ptr(), proj.stride(0), powers.data_ptr(),
@@ -1514,7 +1537,7 @@ def gated_delta_scan(conv, araw, braw, gate, A_log, dt_bias, normw, state, ent, 
     assert H % G == 0
     _scan_state_ok(state, H, D, V, ent)
     if _chunked(ent_host):
-        vent, cent = (t_.to(conv.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, conv.device)
         NV = vent.shape[0]
         cs = torch.empty(NV, H, D, V, device=conv.device, dtype=torch.float32)
         ct = torch.empty(NV, H, D, D, device=conv.device, dtype=torch.float32)
@@ -1588,7 +1611,7 @@ def mlstm_scan(proj, bi, bf, cap: float, normw, state, mstate, ent, ent_host, ou
     vent = cent = cs = cd = None
     NV = 0
     if _chunked(ent_host):
-        vent, cent = (t_.to(proj.device) for t_ in scan_chunks(ent_host, SCAN_CHUNK))
+        vent, cent = chunk_tables(ent_host, SCAN_CHUNK, proj.device)
         NV = vent.shape[0]
         cs = torch.empty(NV, H, D, V + 1, device=proj.device, dtype=torch.float32)
         cd = torch.empty(NV, H, D, device=proj.device, dtype=torch.float32)
