@@ -20,10 +20,10 @@
 // gate: head h of row r leaves multiplied by sigmoid(gate[r, h]), or (gate_pc) its channel c by
 // sigmoid(gate[r, h * V + c]).  Optional pooled blocks (`blk`): beside the tokens of the window a
 // row sees one key and value for every block of P tokens that lies wholly before the window,
-// (i - win + 1) / P of them, stored in a pool of their own (the row of the block with last token
-// t: the page that holds t times ceil(page / P), plus (t % page) / P); blocks and tokens share
-// the softmax.  One block per (query row, key/value head): the heads of the group share the
-// key and value tiles, which stream through LDS with an online softmax.
+// (i - win + 1) / P of them, kept in a pool of their own (the row of the block with last token
+// t: the page that holds t times ceil(page / P), plus (t % page) / P), and weighs
+// them in the softmax of its tokens.  One block per (query row, key/value head): the heads of the
+// group share the key and value tiles, which stream through LDS with an online softmax.
 //
 // rope_rows_k: turns the channel pairs (2i, 2i+1) of a stretch of every head by pos * inv_freq[i]
 // and writes them to another place (its own rows or scattered ones).  qtemp_kv_store_k: the

@@ -14,8 +14,8 @@ is wrapped around the residual stream,
                                                              one weight for all channels; a
                                                              stretch of layers may run several
                                                              passes (``loop``)
-    "post"        x <- x + norm(f(x))                        the sublayers read x itself, a
-                                                             norm on what they produce only
+    "post"        x <- x + norm(f(x))                        no norm on the way in, one on
+                                                             the way out
 
 and whether learned absolute positions are added to the token embedding.  Mixers:
 
