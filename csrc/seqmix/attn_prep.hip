@@ -1,11 +1,12 @@
 // Input passes of grouped-query attention behind short convolutions, and the pooled blocks of
 // its key/value pool.
 //
-// conv_rope_norm_store_k: one projection buffer holds q (H heads x D) | k (G x D) | v (G x V) of
-// every row.  Each channel goes through a causal convolution over the sequence's last K
+// conv_rope_norm_store_k: one projection buffer holds q (H heads x D) | k (G x D) | v (GV x V) of
+// every row (differential attention has two q / k heads, its maps, per value head; a layer that
+// reads another layer's keys and values has queries only, G = GV = 0).  Each channel goes through a causal convolution over the sequence's last K
 // projected values (those before the portion come from the slot's saved tail, or are zero before
 // position 0); nrot channel pairs (i, i + nrot) of every q / k head are turned by the angle
-// pos * inv_freq[i]; q and k heads are divided by their root mean square, sqrt(mean x^2 + eps);
+// pos * inv_freq[i]; q and k heads are divided by their root mean square, sqrt(mean x^2 + eps) (`norm`);
 // q also takes a factor per head (`temp`), which stands for a factor on that head's scores.  q
 // goes to its own buffer, k | v to the row of the paged pool that the token owns.  Convolution,
 // angles, rotation and norm are fp32.  One wavefront per (row, head).
@@ -22,7 +23,7 @@ using namespace sm;
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, int V,
+conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V, int norm,
                        const float* __restrict__ cw, int K, float* tail,
                        const int* __restrict__ ent, const int* __restrict__ row_ent,
                        const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
@@ -32,12 +33,12 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D,
   extern __shared__ float smem[];
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int hh = blockIdx.y * 4 + wave;                 // q heads, then k heads, then v heads
-  const bool on = hh < H + 2 * G;
+  const bool on = hh < H + G + GV;
   const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
   const int hd = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
   const int n = kind == 2 ? V : D;
   const int c0 = kind == 0 ? hd * D : kind == 1 ? (H + hd) * D : (H + G) * D + hd * V;
-  const int C = (H + G) * D + G * V, W = G * (D + V);
+  const int C = (H + G) * D + GV * V, W = G * D + GV * V;
   float* s = smem + wave * LDS;
   const int e = row_ent[r];
   const Entry en = load_entry(ent, e);
@@ -79,9 +80,11 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D,
       s[j + nrot] = y;
       ss += x * x + y * y;
     }
-    for (int i = 2 * nrot + lane; i < n; i += 64) ss += s[i] * s[i];
-    ss = wave_sum(ss);
-    rs = 1.0f / sqrtf(ss / (float)n + eps);
+    if (norm) {
+      for (int i = 2 * nrot + lane; i < n; i += 64) ss += s[i] * s[i];
+      ss = wave_sum(ss);
+      rs = 1.0f / sqrtf(ss / (float)n + eps);
+    }
     if (kind == 0 && temp) rs *= temp[hd];
   }
   // another lane may have turned the value this lane stores
@@ -111,7 +114,7 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D,
 #define RT 8
 template <typename T, int KT>
 __global__ void __launch_bounds__(256)
-conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int D, int V,
+conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V, int norm,
                       const float* __restrict__ cw, const float* __restrict__ tail,
                       const int* __restrict__ ent, const int* __restrict__ row_ent,
                       const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
@@ -129,9 +132,9 @@ conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int D, 
     smem[2 * idx + 1] = sn;
   }
   __syncthreads();
-  const int C = (H + G) * D + G * V, W = G * (D + V);
+  const int C = (H + G) * D + GV * V, W = G * D + GV * V;
   const int hh = blockIdx.y * 4 + wave;
-  if (hh < H + 2 * G) {
+  if (hh < H + G + GV) {
     const int kind = hh < H ? 0 : hh < H + G ? 1 : 2;
     const int hd = kind == 0 ? hh : kind == 1 ? hh - H : hh - H - G;
     const int n = kind == 2 ? V : D;
@@ -198,9 +201,12 @@ conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int D, 
           s[j + nrot] = y;
           ss += x * x + y * y;
         }
-        for (int k = 2 * nrot + lane; k < n; k += 64) ss += s[k] * s[k];
-        ss = wave_sum(ss);
-        rs = 1.0f / sqrtf(ss / (float)n + eps) * tq;
+        rs = tq;
+        if (norm) {
+          for (int k = 2 * nrot + lane; k < n; k += 64) ss += s[k] * s[k];
+          ss = wave_sum(ss);
+          rs = 1.0f / sqrtf(ss / (float)n + eps) * tq;
+        }
       }
       __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
       for (int k = lane; k < n; k += 64) stf(dst, k, s[k] * rs);
@@ -242,7 +248,7 @@ extern "C" {
 
 // rows: several rows per workgroup (3 or 4 taps, head sizes up to 256); the tails and blocks of
 // every portion, also of single tokens, are then left to other kernels
-int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, int V,
+int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int GV, int D, int V, int norm,
                                 const float* cw, int K, float* tail, const int* ent,
                                 const int* row_ent, const float* inv_freq, int nrot,
                                 const float* temp, float eps, const int* pos,
@@ -250,7 +256,7 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, 
                                 int P, const int* bt, int max_pages, int page, int R, int rows,
                                 int f32, hipStream_t st) {
   if (R <= 0) return 0;
-  if (H < 1 || G < 1 || D < 1 || V < 1 || K < 1 || nrot < 0 || 2 * nrot > D || page < 1 ||
+  if (H < 1 || G < 0 || GV < 0 || (G + GV > 0 && !pool) || D < 1 || V < 1 || K < 1 || nrot < 0 || 2 * nrot > D || page < 1 ||
       (blk && P < 1))
     return (int)hipErrorInvalidValue;
   const int LDS = D > V ? D : V;
@@ -258,10 +264,10 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, 
   const size_t shm = ((size_t)RT * nrot * 2 + 4 * LDS) * 4;
   if (rows) {
     if ((K != 4 && K != 3) || LDS > 256 || shm > 64 * 1024) return (int)hipErrorInvalidValue;
-    dim3 gr((R + RT - 1) / RT, (H + 2 * G + 3) / 4);
+    dim3 gr((R + RT - 1) / RT, (H + G + GV + 3) / 4);
 #define CRN(KT)                                                                                   \
   SM_DISPATCH_T(f32, hipLaunchKernelGGL((conv_rope_norm_rows_k<T, KT>), gr, dim3(256), shm, st,   \
-                                         (const T*)proj, ldp, H, G, D, V, cw, tail, ent, row_ent, \
+                                         (const T*)proj, ldp, H, G, GV, D, V, norm, cw, tail, ent, row_ent, \
                                          inv_freq, nrot, temp, eps, pos, cache_rows, (T*)pool,    \
                                          (T*)q_out, ldq, R, LDS))
     if (K == 4) CRN(4);
@@ -269,9 +275,9 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int D, 
 #undef CRN
     return (int)hipGetLastError();
   }
-  dim3 grid(R, (H + 2 * G + 3) / 4);
+  dim3 grid(R, (H + G + GV + 3) / 4);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(conv_rope_norm_store_k<T>, grid, dim3(256),
-                                         (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, D, V,
+                                         (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, GV, D, V, norm,
                                          cw, K, tail, ent, row_ent, inv_freq, nrot, temp, eps, pos,
                                          cache_rows, (T*)pool, (T*)q_out, ldq, (T*)blk, P, bt,
                                          max_pages, page, LDS));

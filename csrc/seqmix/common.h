@@ -24,6 +24,9 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf
 __device__ __forceinline__ float softplusf_(float x) {
   return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x)));
 }
+__device__ __forceinline__ float logsigmoidf_(float x) {
+  return fminf(x, 0.0f) - log1pf(expf(-fabsf(x)));
+}
 
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

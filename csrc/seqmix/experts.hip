@@ -6,7 +6,8 @@
 // `groups` contiguous blocks of equal size; a block is ranked by the sum of its two best choice
 // scores or by its best one; experts outside the `keep` best blocks are struck out, and the
 // `top` largest remaining choice scores win (ties: the lower index).  The weights are the
-// winners' s (without the correction), not rescaled.  A token r routed to its k-th expert is slot
+// winners' s (without the correction), as they are or divided by their sum + 1e-20, times a constant.
+// A token r routed to its k-th expert is slot
 // r * top + k; every expert gets the list of its slots (cnt / rows).
 //
 // expert_gemm: for expert e and each of its slots s: out[s] = x[s / x_div] . W_e^T.  Rows are
@@ -48,13 +49,14 @@ __global__ void __launch_bounds__(256)
 group_route_k(const T* __restrict__ h, int ldh, const float* __restrict__ wr, int W, int E, int top,
               int groups, int keep, int score, const float* __restrict__ corr, int gscore,
               int* __restrict__ ids, float* __restrict__ wts, int* __restrict__ cnt,
-              int* __restrict__ rows, int ldr, const float* __restrict__ bias) {
+              int* __restrict__ rows, int ldr, const float* __restrict__ bias, int renorm,
+              float wscale) {
   extern __shared__ float smem[];
   float* sh = smem;          // [W] the row in fp32
   float* ss = sh + W;        // [E] scores (the weights of the chosen)
   float* sc = ss + E;        // [E] choice scores; -inf marks "cannot be chosen (any more)"
   float* sgs = sc + E;       // [groups] group scores
-  float* stop = sgs + groups;   // [top] the chosen logits (score 2)
+  float* stop = sgs + groups;   // [top] the chosen logits (score 2) or scores (renorm)
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
   for (int i = threadIdx.x; i < W; i += blockDim.x) sh[i] = ldf(h, (size_t)r * ldh + i);
   __syncthreads();
@@ -148,8 +150,8 @@ group_route_k(const T* __restrict__ h, int ldh, const float* __restrict__ wr, in
       sc[bi] = -INFINITY;
       int slot = r * top + k;
       ids[slot] = bi;
-      if (score == 2) stop[k] = ss[bi];
-      else wts[slot] = ss[bi];
+      if (score == 2 || renorm) stop[k] = ss[bi];
+      else wts[slot] = ss[bi] * wscale;
       int at = atomicAdd(&cnt[bi], 1);
       rows[(size_t)bi * ldr + at] = slot;
     }
@@ -163,7 +165,12 @@ group_route_k(const T* __restrict__ h, int ldh, const float* __restrict__ wr, in
     float sum = 0.0f;
     for (int k = lane; k < top; k += 64) sum += expf(stop[k] - mx);
     sum = wave_sum(sum);
-    for (int k = lane; k < top; k += 64) wts[r * top + k] = expf(stop[k] - mx) / sum;
+    for (int k = lane; k < top; k += 64) wts[r * top + k] = expf(stop[k] - mx) / sum * wscale;
+  } else if (renorm) {
+    float sum = 0.0f;
+    for (int k = lane; k < top; k += 64) sum += stop[k];
+    sum = wave_sum(sum) + 1e-20f;
+    for (int k = lane; k < top; k += 64) wts[r * top + k] = stop[k] / sum * wscale;
   }
 }
 
@@ -530,8 +537,8 @@ extern "C" {
 // cnt must be zero on entry
 int p2p_sm_group_route(const void* h, int ldh, const float* wr, int R, int W, int E, int top,
                        int groups, int keep, int score, const float* corr, int gscore, int* ids,
-                       float* wts, int* cnt, int* rows, int ldr, const float* bias, int f32,
-                       hipStream_t st) {
+                       float* wts, int* cnt, int* rows, int ldr, const float* bias, int renorm,
+                       float wscale, int f32, hipStream_t st) {
   if (R <= 0) return 0;
   if (E < 1 || groups < 1 || E % groups || keep < 1 || keep > groups || top < 1 ||
       top > keep * (E / groups) || ldr < R * top)
@@ -540,7 +547,7 @@ int p2p_sm_group_route(const void* h, int ldh, const float* wr, int R, int W, in
   if (shm > 64 * 1024) return (int)hipErrorInvalidValue;
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(group_route_k<T>, dim3(R), dim3(256), shm, st,
                                          (const T*)h, ldh, wr, W, E, top, groups, keep, score, corr,
-                                         gscore, ids, wts, cnt, rows, ldr, bias));
+                                         gscore, ids, wts, cnt, rows, ldr, bias, renorm, wscale));
   return (int)hipGetLastError();
 }
 

@@ -23,6 +23,10 @@
 // k = silu(.), v = silu(.); its norm spans all heads of a row, so o leaves in fp32 as it is.  This
 // kernel walks its decode steps and short portions; long ones go through lightning.hip.
 //
+// Gated linear attention is the plain write with a decay per key channel on unchanged projections:
+// q D^-1/2, k, v, and g = sigmoid(z)^(1/tau), formed as exp(logsigmoid(z) / tau), where z is a low-rank
+// projection plus a bias; after the head's norm comes a silu gate.  Long portions go through gla.hip.
+//
 // The value columns of S are independent.  A wavefront covers 16 columns x 4 slices of the key
 // index; lane (c, s) keeps rows s*DQ .. s*DQ+DQ-1 of column c in registers (NC columns, 16
 // apart, in the general form of the kernel), and the sums over the key index (S^T k before
@@ -60,6 +64,9 @@ struct ScanArgs {
   // lightning: proj = [q (H*D) | k (H*D) | v (H*V) | ...]; pw fp32 [H, ldw], the powers of every
   // head's decay (column 1 is the decay); out is fp32
   const float* pw; int ldw;
+  // gated linear attention: proj = [q (H*D) | k (H*D) | v (H*V) | gate (H*V) | ...], decay logits
+  // z = sum_l low[l] w_a2[i][l] + dt_bias[i]: `low` is `rank` columns of proj from column `low0`
+  const void* wa2; int low0, rank; float inv_tau;
   int VS;   // value columns of the state: V, or V + 1 with the normaliser
   // common
   const float* normw; float* state; const int* ent; void* out; int ldo;
@@ -75,9 +82,9 @@ struct ScanArgs {
   float* chunk_trans;   // [chunks, H, D, D]
 };
 
-template <typename T, int DQ, int KIND, int NC>   // KIND 0: plain write (HGRN2), 1: delta rule, 2: matrix memory, 3: lightning
+template <typename T, int DQ, int KIND, int NC>   // KIND 0: plain write (HGRN2), 1: delta rule, 2: matrix memory, 3: lightning, 4: gated linear attention
 __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
-  constexpr bool DELTA = KIND == 1, MEM = KIND == 2, LIGHT = KIND == 3;
+  constexpr bool DELTA = KIND == 1, MEM = KIND == 2, LIGHT = KIND == 3, GLA = KIND == 4;
   constexpr int DKP = 4 * DQ;   // padded key index (zero filled in LDS)
   constexpr int WC = 16 * NC;   // columns per wavefront: a lane keeps NC columns, 16 apart
   const int H = a.H, D = a.D, V = a.V, VS = a.VS, CT = a.CT, mode = a.mode;
@@ -136,7 +143,7 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
   if (!DELTA && mode == 1)
     for (int i = threadIdx.x; i < DKP; i += blockDim.x) sP[i] = 1.0f;
   const float negA = DELTA ? -expf(a.A_log[h]) : 0.0f;
-  const float qscale = (DELTA || MEM) ? 1.0f / sqrtf((float)D) : 1.0f;
+  const float qscale = (DELTA || MEM || GLA) ? 1.0f / sqrtf((float)D) : 1.0f;
   for (int t0 = 0; t0 < en.n; t0 += CT) {
     const int ct = min(CT, en.n - t0);
     for (int idx = threadIdx.x; idx < ct * DKP; idx += blockDim.x) {
@@ -160,6 +167,14 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
           vq = qr * sigmoidf_(qr);
           vk = kr * sigmoidf_(kr);
           vg = a.pw[(size_t)h * a.ldw + 1];
+        } else if (GLA) {
+          vq = ldf(proj, row * a.ldp + h * D + i) * qscale;
+          vk = ldf(proj, row * a.ldp + H * D + h * D + i);
+          const T* w = (const T*)a.wa2 + (size_t)(h * D + i) * a.rank;
+          const T* lo = proj + row * a.ldp + a.low0;
+          float z = 0.0f;
+          for (int l = 0; l < a.rank; l++) z += ldf(lo, l) * ldf(w, l);
+          vg = expf(logsigmoidf_(z + a.dt_bias[h * D + i]) * a.inv_tau);
         } else {
           float qr = ldf(proj, row * a.ldp + h * D + i);
           vq = qr * sigmoidf_(qr);
@@ -317,6 +332,10 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
         } else {
           y = so[t * VP + i] * rs * a.normw[i];
           if (DELTA) y *= sigmoidf_(ldf(gate, row * a.ldg + h * V + i));
+          if (GLA) {
+            const float gt = ldf(proj, row * a.ldp + 2 * H * D + H * V + h * V + i);
+            y *= gt * sigmoidf_(gt);
+          }
         }
         stf(out, row * a.ldo + h * V + i, y);
       }
@@ -435,10 +454,6 @@ dense_chain_k(float* __restrict__ cs, const float* __restrict__ trans, float* __
 // m through the composites of the block's wavefronts; then every lane applies its prefix map
 // to the m at its group's start.  Any rounding of m only moves the scale on which S and n are
 // kept: the coefficients are formed from the same m values, so S e^m and n e^m stay exact.
-__device__ __forceinline__ float logsigmoidf_(float x) {
-  return fminf(x, 0.0f) - log1pf(expf(-fabsf(x)));
-}
-
 template <typename T>
 __global__ void __launch_bounds__(1024)
 mlstm_gates_k(const T* __restrict__ proj, int ldp, int off_i, int off_f,
@@ -566,6 +581,19 @@ int p2p_sm_lightning_scan(const void* proj, int ldp, const float* pw, int ldw, f
   a.state = state; a.ent = ent; a.out = out; a.ldo = ldo;
   a.H = H; a.G = H; a.D = D; a.V = V;
   return launch_scan<3>(a, E, f32, st);
+}
+
+// gated linear attention, portions in one pass (wa2 [H*D, rank] in the activation type, za the bias)
+int p2p_sm_gla_scan(const void* proj, int ldp, int low0, int rank, const void* wa2, const float* za,
+                    float inv_tau, const float* normw, float* state, const int* ent, int E, void* out,
+                    int ldo, int H, int D, int V, float eps, float out_scale, int f32,
+                    hipStream_t st) {
+  if (rank < 1) return (int)hipErrorInvalidValue;
+  ScanArgs a = {};
+  a.proj = proj; a.ldp = ldp; a.low0 = low0; a.rank = rank; a.wa2 = wa2; a.dt_bias = za;
+  a.inv_tau = inv_tau; a.normw = normw; a.state = state; a.ent = ent; a.out = out; a.ldo = ldo;
+  a.H = H; a.G = H; a.D = D; a.V = V; a.eps = eps; a.out_scale = out_scale;
+  return launch_scan<4>(a, E, f32, st);
 }
 
 int p2p_sm_hgrn2_scan(const void* proj, int ldp, const float* lower, const float* fb,

@@ -7,7 +7,7 @@
 // separated, a weight per channel of the row) or, `per_head`, one per head and a weight of D
 // channels that the heads share -- and nrot channel pairs of every head, (2i, 2i+1) or, `half`,
 // (i, i + nrot), are turned by the angle pos * inv_freq[i]:
-// (a, b) -> (a cos - b sin, b cos + a sin).  q goes to its own buffer, k | v to the row of the
+// (a, b) -> (a cos - b sin, b cos + a sin), cos and sin times `rm`.  q goes to its own buffer, k | v to the row of the
 // paged pool that the token owns; a layer that reads another layer's keys and values passes no
 // pool and only its queries are prepared.  Norm, angle and rotation are fp32.
 //
@@ -22,7 +22,10 @@
 // row sees one key and value for every block of P tokens that lies wholly before the window,
 // (i - win + 1) / P of them, kept in a pool of their own (the row of the block with last token
 // t: the page that holds t times ceil(page / P), plus (t % page) / P), and weighs
-// them in the softmax of its tokens.  One block per (query row, key/value head): the heads of the
+// them in the softmax of its tokens; or the first `keep` tokens of the sequence, whatever their
+// distance.  With maps = 2 every query and key head has two maps of D channels, [map 1 | map 2] per
+// head, on the same values: each map is an attention of its own and its result goes to place
+// head * 2 + map of the output row (fp32; diff_combine_k takes their difference).  One block per (query row, key head): the heads of the
 // group share the key and value tiles, which stream through LDS with an online softmax.
 //
 // rope_rows_k: turns the channel pairs (2i, 2i+1) of a stretch of every head by pos * inv_freq[i]
@@ -38,7 +41,7 @@ qk_norm_rope_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, i
                      const float* __restrict__ qw, const float* __restrict__ kw,
                      const float* __restrict__ inv_freq, int nrot, const int* __restrict__ pos,
                      const int* __restrict__ cache_rows, T* __restrict__ pool, float eps,
-                     T* __restrict__ q_out, int ldq, int per_head, int half) {
+                     T* __restrict__ q_out, int ldq, int per_head, int half, float rm) {
   __shared__ float red[16];
   const int r = blockIdx.x;
   const int nq = H * D, nk = G * D, nv = G * V;
@@ -87,6 +90,8 @@ qk_norm_rope_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, i
       float a = ldf(src, ca) * rs * w[ca], b = ldf(src, cb) * rs * w[cb];
       float sn, cs;
       sincosf(p * inv_freq[j], &sn, &cs);
+      sn *= rm;
+      cs *= rm;
       stf(dst, ca, a * cs - b * sn);
       stf(dst, cb, b * cs + a * sn);
     }
@@ -100,7 +105,7 @@ template <typename T>
 __global__ void rope_rows_k(const T* __restrict__ src, int lds_, int heads, int src_hs,
                             const float* __restrict__ inv_freq, int nrot,
                             const int* __restrict__ pos, const int* __restrict__ out_rows,
-                            T* __restrict__ dst, long ldd, long dst_hs) {
+                            T* __restrict__ dst, long ldd, long dst_hs, float rm) {
   const int r = blockIdx.x;
   const float p = (float)pos[r];
   const long ro = out_rows ? out_rows[r] : r;
@@ -112,6 +117,8 @@ __global__ void rope_rows_k(const T* __restrict__ src, int lds_, int heads, int 
     float a = ldf(s, (size_t)h * src_hs + 2 * i), b = ldf(s, (size_t)h * src_hs + 2 * i + 1);
     float sn, cs;
     sincosf(p * inv_freq[i], &sn, &cs);
+    sn *= rm;
+    cs *= rm;
     stf(d, (size_t)(h * dst_hs + 2 * i), a * cs - b * sn);
     stf(d, (size_t)(h * dst_hs + 2 * i + 1), b * cs + a * sn);
   }
@@ -130,10 +137,11 @@ latent_prep_k(const T* __restrict__ proj, int ldp, int nq, int nc, int nr,
               const float* __restrict__ qw, const float* __restrict__ cw,
               const float* __restrict__ inv_freq, int nrot, const int* __restrict__ pos,
               const int* __restrict__ cache_rows, T* __restrict__ pool, float eps,
-              T* __restrict__ cq, int ldq) {
+              T* __restrict__ cq, int ldq, float rm) {
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* row = proj + (size_t)r * ldp;
   T* crow = pool + (size_t)cache_rows[r] * (nc + nr);
+  if (wave == 0 && nq == 0) return;   // queries without a latent
   if (wave < 2) {
     const T* src = row + (wave ? nq : 0);
     const int n = wave ? nc : nq;
@@ -175,6 +183,8 @@ latent_prep_k(const T* __restrict__ proj, int ldp, int nq, int nc, int nr,
     float a = ldf(src, 2 * i), b = ldf(src, 2 * i + 1);
     float sn, cs;
     sincosf(p * inv_freq[i], &sn, &cs);
+    sn *= rm;
+    cs *= rm;
     stf(dst, 2 * i, a * cs - b * sn);
     stf(dst, 2 * i + 1, b * cs + a * sn);
   }
@@ -199,21 +209,22 @@ __global__ void qtemp_kv_store_k(const T* __restrict__ proj, int ldp, int nq, in
 #define WA_THREADS 256
 #define WA_ACC 16      // (head, value channel) pairs per thread at most
 
-template <typename T>
+template <typename T, typename TO>
 __global__ void __launch_bounds__(WA_THREADS)
 window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
               const int* __restrict__ bt, int max_pages, const int* __restrict__ row_ent,
               const int* __restrict__ pos, const float* __restrict__ sink, float scale, int win,
-              T* __restrict__ out, int ldo, int H, int G, int D, int V, int page, int TK,
+              TO* __restrict__ out, int ldo, int H, int G, int D, int V, int page, int TK,
               float out_scale, int HB, float cap, const float* __restrict__ r1,
               const float* __restrict__ r2, const T* __restrict__ gate, int ldg, int gate_pc,
-              const T* __restrict__ blk, int P) {
+              const T* __restrict__ blk, int P, int keep, int maps) {
   extern __shared__ float smem[];
-  // a block takes up to HB query heads of one key/value head (all of them when they fit)
+  // a block takes up to HB query heads of one key head (all of them when they fit)
   const int nhb = (H / G + HB - 1) / HB;
-  const int g = blockIdx.y / nhb, hb0 = (blockIdx.y % nhb) * HB;
+  const int gk = blockIdx.y / nhb, hb0 = (blockIdx.y % nhb) * HB;
+  const int g = gk / maps, map = gk % maps;
   const int h0 = g * (H / G) + hb0, HG = min(HB, H / G - hb0);
-  const int ldk = D + 1, ldv = V + 1, ldpool = G * (D + V);
+  const int ldk = D + 1, ldv = V + 1, ldpool = G * (maps * D + V);
   float* sq = smem;                      // [HB][D]
   float* sk = sq + HB * D;               // [TK][D + 1]
   float* sv = sk + TK * ldk;             // [TK][V + 1]
@@ -227,18 +238,19 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
   const int w_lo = max(0, p - win + 1);
   // keys are walked as pooled blocks 0 .. nb-1 followed by tokens w_lo .. p: place u of that list
   // is token u + w_lo - nb from place nb on
-  const int nb = blk ? w_lo / P : 0, shift = w_lo - nb, SB = blk ? (page + P - 1) / P : 1;
+  // (with kept tokens: those before w_lo come first instead)
+  const int nb = blk ? w_lo / P : min(keep, w_lo), shift = w_lo - nb, SB = blk ? (page + P - 1) / P : 1;
   const int last = p - shift;
   auto key_row = [&](int u) {
-    if (u < nb) {
+    if (blk && u < nb) {
       const int t = u * P + P - 1;
       return blk + ((size_t)pages[t / page] * SB + (t % page) / P) * ldpool;
     }
-    const int j = u + shift;
+    const int j = u < nb ? u : u + shift;
     return pool + ((size_t)pages[j / page] * page + (j % page)) * ldpool;
   };
   for (int idx = tid; idx < HG * D; idx += WA_THREADS)
-    sq[idx] = ldf(q, (size_t)r * ldq + (size_t)h0 * D + idx);
+    sq[idx] = ldf(q, (size_t)r * ldq + (size_t)((h0 + idx / D) * maps + map) * D + idx % D);
   if (tid < HG) {
     sm_[tid] = sink ? sink[h0 + tid] : -1e30f;   // no sink: an ordinary softmax
     sl[tid] = sink ? 1.0f : 0.0f;
@@ -252,11 +264,11 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
     __syncthreads();  // previous tile fully consumed (and sq / sm_ / sl initialised)
     for (int idx = tid; idx < nk * D; idx += WA_THREADS) {
       int jj = idx / D, c = idx % D;
-      sk[jj * ldk + c] = ldf(key_row(j0 + jj), (size_t)g * D + c);
+      sk[jj * ldk + c] = ldf(key_row(j0 + jj), (size_t)gk * D + c);
     }
     for (int idx = tid; idx < nk * V; idx += WA_THREADS) {
       int jj = idx / V, c = idx % V;
-      sv[jj * ldv + c] = ldf(key_row(j0 + jj), (size_t)G * D + (size_t)g * V + c);
+      sv[jj * ldv + c] = ldf(key_row(j0 + jj), (size_t)G * maps * D + (size_t)g * V + c);
     }
     __syncthreads();
     for (int idx = tid; idx < HG * TK; idx += WA_THREADS) {
@@ -269,7 +281,10 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
         for (int i = 0; i < D; i++) d += qh[i] * kr[i];
         s = d * scale;
         if (cap > 0.0f) s = cap * tanhf(s / cap);
-        if (r1) s -= r1[h0 + h] * log1pf(r2[h0 + h] * (float)(last - (j0 + jj)));
+        if (r1) {
+          const int u = j0 + jj;
+          s -= r1[h0 + h] * log1pf(r2[h0 + h] * (float)(p - (u < nb ? u : u + shift)));
+        }
       }
       sp[idx] = s;
     }
@@ -313,47 +328,77 @@ window_attn_k(const T* __restrict__ q, int ldq, const T* __restrict__ pool,
       float o = acc[a] / sl[h] * out_scale;
       if (gate)
         o *= sigmoidf_(ldf(gate, (size_t)r * ldg + (gate_pc ? (size_t)h0 * V + idx : h0 + h)));
-      stf(out, (size_t)r * ldo + (size_t)h0 * V + idx, o);
+      stf(out, (size_t)r * ldo + (size_t)((h0 + h) * maps + map) * V + idx % V, o);
     }
   }
 }
 
+// Difference of the two maps of differential attention, a fp32 [R, H, 2, V] -> out [R, H*V]:
+// o = a_1 - lam a_2, divided by sqrt(mean(o^2) + eps) over the head's V channels, times out_scale.
+// One wavefront per (row, head).
+template <typename T>
+__global__ void __launch_bounds__(256)
+diff_combine_k(const float* __restrict__ a, int lda, T* __restrict__ out, int ldo, int H, int V, float lam,
+               float eps, float out_scale) {
+  const int r = blockIdx.x, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (h >= H) return;
+  const float* s = a + (size_t)r * lda + (size_t)h * 2 * V;
+  float ss = 0.0f;
+  for (int c = lane; c < V; c += 64) {
+    const float o = s[c] - lam * s[V + c];
+    ss += o * o;
+  }
+  ss = wave_sum(ss);
+  const float rs = out_scale / sqrtf(ss / (float)V + eps);
+  for (int c = lane; c < V; c += 64)
+    stf(out, (size_t)r * ldo + (size_t)h * V + c, (s[c] - lam * s[V + c]) * rs);
+}
+
 extern "C" {
+
+int p2p_sm_diff_combine(const float* a, int lda, void* out, int ldo, int R, int H, int V, float lam,
+                        float eps, float out_scale, int f32, hipStream_t st) {
+  if (R <= 0) return 0;
+  if (H < 1 || V < 1) return (int)hipErrorInvalidValue;
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL(diff_combine_k<T>, dim3(R, (H + 3) / 4), dim3(256), 0, st, a, lda,
+                                         (T*)out, ldo, H, V, lam, eps, out_scale));
+  return (int)hipGetLastError();
+}
 
 int p2p_sm_qk_norm_rope_store(const void* proj, int ldp, int H, int G, int D, int V,
                               const float* qw, const float* kw, const float* inv_freq, int nrot,
                               const int* pos, const int* cache_rows, void* pool, float eps,
-                              void* q_out, int ldq, int R, int per_head, int half, int f32,
-                              hipStream_t st) {
+                              void* q_out, int ldq, int R, int per_head, int half, float rm,
+                              int f32, hipStream_t st) {
   if (R <= 0) return 0;
   if (H < 1 || G < 1 || D < 1 || V < 1 || nrot < 0 || 2 * nrot > D) return (int)hipErrorInvalidValue;
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(qk_norm_rope_store_k<T>, dim3(R), dim3(256), 0, st,
                                          (const T*)proj, ldp, H, G, D, V, qw, kw, inv_freq, nrot,
                                          pos, cache_rows, (T*)pool, eps, (T*)q_out, ldq, per_head,
-                                         half));
+                                         half, rm));
   return (int)hipGetLastError();
 }
 
 int p2p_sm_rope_rows(const void* src, int lds_, int heads, int src_hs, const float* inv_freq,
                      int nrot, const int* pos, const int* out_rows, void* dst, long ldd,
-                     long dst_hs, int R, int f32, hipStream_t st) {
+                     long dst_hs, int R, float rm, int f32, hipStream_t st) {
   if (R <= 0 || heads <= 0 || nrot <= 0) return 0;
   int threads = heads * nrot >= 256 ? 256 : 64;
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(rope_rows_k<T>, dim3(R), dim3(threads), 0, st,
                                          (const T*)src, lds_, heads, src_hs, inv_freq, nrot, pos,
-                                         out_rows, (T*)dst, ldd, dst_hs));
+                                         out_rows, (T*)dst, ldd, dst_hs, rm));
   return (int)hipGetLastError();
 }
 
 int p2p_sm_latent_prep(const void* proj, int ldp, int nq, int nc, int nr, const float* qw,
                        const float* cw, const float* inv_freq, int nrot, const int* pos,
                        const int* cache_rows, void* pool, float eps, void* cq, int ldq, int R,
-                       int f32, hipStream_t st) {
+                       float rm, int f32, hipStream_t st) {
   if (R <= 0) return 0;
-  if (nq < 1 || nc < 1 || nr < 0 || nrot < 0 || 2 * nrot > nr) return (int)hipErrorInvalidValue;
+  if (nq < 0 || (nq > 0 && (!qw || !cq)) || nc < 1 || nr < 0 || nrot < 0 || 2 * nrot > nr) return (int)hipErrorInvalidValue;
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(latent_prep_k<T>, dim3(R), dim3(192), 0, st,
                                          (const T*)proj, ldp, nq, nc, nr, qw, cw, inv_freq, nrot,
-                                         pos, cache_rows, (T*)pool, eps, (T*)cq, ldq));
+                                         pos, cache_rows, (T*)pool, eps, (T*)cq, ldq, rm));
   return (int)hipGetLastError();
 }
 
@@ -372,10 +417,11 @@ int p2p_sm_window_attn(const void* q, int ldq, const void* pool, const int* bt, 
                        const int* row_ent, const int* pos, const float* sink, float scale, int win,
                        void* out, int ldo, int R, int H, int G, int D, int V, int page,
                        float out_scale, float cap, const float* r1, const float* r2,
-                       const void* gate, int ldg, int gate_pc, const void* blk, int P, int f32,
-                       hipStream_t st) {
+                       const void* gate, int ldg, int gate_pc, const void* blk, int P, int keep,
+                       int maps, int f32, hipStream_t st) {
   if (R <= 0) return 0;
   if (H < 1 || G < 1 || H % G || D < 1 || V < 1 || win < 1 || (r1 && !r2) || cap < 0.0f ||
+      keep < 0 || (keep && blk) || maps < 1 || maps > 2 || (maps == 2 && (sink || gate || blk)) ||
       (blk && (P < 1 || r1)))   // a distance penalty needs positions, which blocks do not have
     return (int)hipErrorInvalidValue;
   int HG = H / G, TK = WA_TK, HB = HG;
@@ -390,12 +436,16 @@ int p2p_sm_window_attn(const void* q, int ldq, const void* pool, const int* bt, 
   while (TK > 2 && lds(TK, HB) > 64 * 1024) TK /= 2;
   if ((long)HB * V > (long)WA_ACC * WA_THREADS || lds(TK, HB) > 64 * 1024)
     return (int)hipErrorInvalidValue;
-  dim3 grid(R, G * ((HG + HB - 1) / HB));
-  SM_DISPATCH_T(f32, hipLaunchKernelGGL(window_attn_k<T>, grid, dim3(WA_THREADS), lds(TK, HB), st,
-                                         (const T*)q, ldq, (const T*)pool, bt, max_pages, row_ent,
-                                         pos, sink, scale, win, (T*)out, ldo, H, G, D, V, page, TK,
-                                         out_scale, HB, cap, r1, r2, (const T*)gate, ldg, gate_pc,
-                                         (const T*)blk, P));
+  dim3 grid(R, G * maps * ((HG + HB - 1) / HB));
+#define WAK(TO)                                                                                     \
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL((window_attn_k<T, TO>), grid, dim3(WA_THREADS), lds(TK, HB), st, \
+                                         (const T*)q, ldq, (const T*)pool, bt, max_pages, row_ent,  \
+                                         pos, sink, scale, win, (TO*)out, ldo, H, G, D, V, page, TK, \
+                                         out_scale, HB, cap, r1, r2, (const T*)gate, ldg, gate_pc,  \
+                                         (const T*)blk, P, keep, maps))
+  if (maps == 2) WAK(float);   // the maps meet in diff_combine_k
+  else WAK(T);
+#undef WAK
   return (int)hipGetLastError();
 }
 

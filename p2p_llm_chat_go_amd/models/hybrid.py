@@ -16,6 +16,11 @@ is wrapped around the residual stream,
                                                              passes (``loop``)
     "post"        x <- x + norm(f(x))                        no norm on the way in, one on
                                                              the way out
+    "streams"     x_t <- sum_s M[s, t] x_s + c_t f(norm(sum_s a_s x_s))
+                                                             hyper-connections: several residual
+                                                             streams that a sublayer reads as a
+                                                             weighted sum and writes all at once;
+                                                             the norm is a dynamic tanh
 
 and whether learned absolute positions are added to the token embedding.  Mixers:
 
@@ -53,11 +58,21 @@ and whether learned absolute positions are added to the token embedding.  Mixers
                         channel and N states per channel;
   ``lightning``         linear attention with one constant decay per head, silu on q, k, v, one
                         norm over all heads and a sigmoid gate;
-  ``parallel``          two mixers side by side on the same input, summed with fixed scales.
+  ``diff_attention``    differential attention behind short convolutions: two attention maps per head on
+                        the same values, their weighted difference normed per head; sliding window
+                        that keeps the first tokens; may borrow an earlier layer's keys and values;
+  ``direct_latent_attention``  ``rope_latent_attention`` with queries projected straight from the input
+                        and no gate;
+  ``gla``               gated linear attention: a decay per key channel, sigmoid(low-rank)^(1/tau),
+                        a norm per head and a silu gate;
+  ``parallel``          two mixers side by side on the same input, summed with fixed scales (window
+                        attention and the gated delta rule unless the config or a subclass says
+                        otherwise: ``parallel_gla`` takes ``attention`` and ``gla``).
 
 Feed-forwards: ``dense`` (silu-gated, or the clamped gated unit when the config gives a
-limit), ``moe`` (sigmoid router, choice limited to the best groups of experts), ``moe_softmax``
-and ``moe_top`` (biased router, softmax over the chosen logits, silu-gated experts, shared expert).
+limit), ``moe`` (sigmoid router, choice limited to the best groups of experts), ``moe_softmax``,
+``moe_top`` (biased router, softmax over the chosen logits, silu-gated experts, shared expert) and
+``moe_group`` (softmax router limited to the best groups, weights rescaled, experts as ``moe_top``).
 A design may give a config's ``type`` / ``kind`` names a meaning of its own (``Design.mixers``,
 ``Design.ff``).
 
@@ -71,7 +86,10 @@ squared-relu experts behind a softmax router.  "Tarunex" stacks ``biased_attenti
 the two-norm parallel form with ``moe_top`` feed-forwards, repeats a stretch of layers, scales
 its embedding and scales and caps its logits.  "Rasepel" stacks ``mamba1``, ``conv_attention``
 (its config's "attention") and ``lightning`` layers in the post-norm form with clamped dense
-feed-forwards, scales its embedding and reads its logits off the embedding table.  A checkpoint is a ``config.json`` whose
+feed-forwards, scales its embedding and reads its logits off the embedding table.  "Nosuzen" stacks
+``diff_attention``, ``direct_latent_attention`` and ``parallel_gla`` layers (its config's "attention",
+"latent_attention" and "parallel") with ``moe_group`` feed-forwards on hyper-connected streams.
+A checkpoint is a ``config.json`` whose
 ``architecture`` names the design and one safetensors file (``load_dir``).
 
 One ``forward`` serves every step: a flat list of token rows cut into entries (portions of
@@ -106,7 +124,7 @@ class LayerSpec:
 @dataclasses.dataclass(frozen=True)
 class Design:
     block: str                # how sublayers sit on the residual stream: "sandwich" | "gated_post" |
-                              # "parallel" | "parallel2" | "post"
+                              # "parallel" | "parallel2" | "post" | "streams"
     positions: str | None     # "learned": a position table is added to the embedding
     norm_offset: float = 0.0  # block and final norm weights are stored minus this (1: around zero)
     ff: tuple = ()            # (config kind, FEEDFORWARDS key) where the two differ
@@ -128,7 +146,10 @@ DESIGNS = {"Regesun": Design("sandwich", "learned"), "Rotutar": Design("gated_po
                              mixers=(("latent_attention", "rope_latent_attention"),
                                      ("attention", "biased_attention"))),
            "Rasepel": Design("post", None, norm_offset=1.0, tied_head=True,
-                             mixers=(("attention", "conv_attention"),))}
+                             mixers=(("attention", "conv_attention"),)),
+           "Nosuzen": Design("streams", None, ff=(("moe", "moe_group"),),
+                             mixers=(("attention", "diff_attention"), ("parallel", "parallel_gla"),
+                                     ("latent_attention", "direct_latent_attention")))}
 NO_POS_LIMIT = 1 << 30
 
 
@@ -148,6 +169,7 @@ class HybridConfig:
     logit_softcap: float = 0.0
     logit_scale: float = 1.0
     embed_scale: float = 1.0
+    streams: int = 1            # residual streams (hyper-connections)
     loop: tuple | None = None   # (start, stop, times): layers start .. stop-1 run `times` passes
 
     @property
@@ -202,7 +224,10 @@ class HybridConfig:
                                  % (loop[0], loop[1] - 1, loop[2], len(layers)))
             if DESIGNS[design].block != "parallel2":
                 raise ValueError("design %s does not repeat layers" % design)
-        return cls(name=name or design.lower(), width=width,
+        streams = int(c.get("streams", 1))
+        if streams < 1 or (streams > 1 and DESIGNS[design].block != "streams"):
+            raise ValueError("design %s with %d residual streams" % (design, streams))
+        return cls(name=name or design.lower(), width=width, streams=streams,
                    vocab=int(c["vocab"]), layers=layers, eps=float(c["norm"]["eps"]),
                    max_pos=max_pos, bos_id=int(c.get("bos_token_id", 1)),
                    eos_ids=eos, design=design, norm_groups=groups,
@@ -232,6 +257,8 @@ class HybridConfig:
             d["logit_scale"] = self.logit_scale
         if self.embed_scale != 1.0:
             d["embedding"] = {"scale": self.embed_scale}
+        if self.traits.block == "streams":
+            d["streams"] = self.streams
         if self.loop:
             d["loop"] = dict(zip(("start", "stop", "times"), self.loop))
         return d
@@ -594,7 +621,8 @@ class WindowAttention(Mixer):
         self.kv_from = int(s["kv_from"]) if s.get("kv_from") is not None else None
         self.H, self.D, self.V = int(s["heads"]), int(s["dim"]), int(s["vdim"])
         self.G = int(s.get("kv_heads", self.H))
-        self.win = int(s["mask"]["size"]) if s.get("mask") else 1 << 30
+        mask = s.get("mask") or {}
+        self.win, self.keep = int(mask.get("size", 1 << 30)), int(mask.get("keep_first", 0))
         self.scale = float(s["scale"]) if "scale" in s else self.D ** -0.5
         rot = s.get("rot")
         self.rot_dims = int(rot["dims"]) if rot else 0
@@ -624,6 +652,7 @@ class WindowAttention(Mixer):
         self.knorm = _vec(get("k.norm"), dev) if own else None
         self.sink = _vec(get("sink"), dev) if self.SINK else None
         self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev, self.rot_scaling)
+        self.rot_mag = sm.rope_magnitude(self.rot_scaling)
         self.wo = get("o").to(dev, dtype).contiguous()
 
     def cache_spec(self):
@@ -644,17 +673,18 @@ class WindowAttention(Mixer):
         q = torch.empty(b.R, H * D, device=proj.device, dtype=proj.dtype)
         sm.qk_norm_rope_store(proj, H, G, D, V, self.qnorm, self.knorm, self.inv_freq, b.pos,
                               b.cache_rows, pool if own else None, self.eps, q,
-                              per_head=self.PER_HEAD, half=self.HALF)
+                              per_head=self.PER_HEAD, half=self.HALF, rm=self.rot_mag)
         units = b.units(sm.window_rows_per_wave(H // G)) if sm.window_mfma_ok(q, pool, D, V) else None
         sm.window_attn(q, pool, b.block_tables, b.row_ent, b.pos, self.sink, self.scale, self.win,
-                       out, PAGE, H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale)
+                       out, PAGE, H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale,
+                       keep=self.keep)
         return out
 
 
 class Attention(WindowAttention):
     """Causal grouped-query attention with an ordinary softmax: per-head query / key norm,
     rotation of the pairs (i, i + dims/2) with optional stretching of long wavelengths
-    (``rot.scaling``), no sink; ``mask`` (a window) stays optional.  ``kv_from: j`` reads layer
+    (``rot.scaling``), no sink; ``mask`` (a window, which may keep the first tokens) stays optional.  ``kv_from: j`` reads layer
     j's keys and values as its cache holds them and projects only queries."""
     kind = "attention"
     PER_HEAD, HALF, SINK = True, True, False
@@ -782,6 +812,84 @@ class ConvAttention(Mixer):
         return out
 
 
+class DiffAttention(Mixer):
+    """Differential attention behind short convolutions (``ops.seqmix.conv_rope_norm_store``,
+    ``window_attn``): every head has two query / key maps of ``dim`` channels on one value; the maps'
+    outputs leave as a_1 - lam a_2, normed per head, times 1 - ``diff``, with one lam per layer,
+    exp(lq1 . lk1) - exp(lq2 . lk2) + diff.  Rotation of the pairs (i, i + dims/2) of every map (``rot``
+    optional), causal window (``mask.size``) that keeps the first ``mask.keep_first`` tokens.
+    ``kv_from: j`` reads layer j's keys and values as its cache holds them and projects (and
+    convolves) only queries."""
+    kind = "diff_attention"
+
+    def _dims(self):
+        s = self.spec
+        self.kv_from = int(s["kv_from"]) if s.get("kv_from") is not None else None
+        self.H, self.D, self.V = int(s["heads"]), int(s["dim"]), int(s["vdim"])
+        self.G, self.K, self.diff = int(s.get("kv_heads", self.H)), int(s["conv"]), float(s["diff"])
+        mask = s.get("mask") or {}
+        self.win, self.keep = int(mask.get("size", 1 << 30)), int(mask.get("keep_first", 0))
+        self.scale = float(s["scale"]) if "scale" in s else self.D ** -0.5
+        rot = s.get("rot")
+        self.rot_dims, self.rot_base = (int(rot["dims"]), float(rot["base"])) if rot else (0, 1.0)
+        self.rot_scaling = dict(rot["scaling"]) if rot and rot.get("scaling") else None
+        if self.H % self.G or self.rot_dims % 2 or self.rot_dims > self.D or self.K < 1 or self.win < 1 \
+                or self.keep < 0:
+            raise ValueError("diff_attention: %d heads / %d kv heads / %d rotated of %d channels / %d taps / "
+                             "window %d + %d" % (self.H, self.G, self.rot_dims, self.D, self.K, self.win,
+                                                 self.keep))
+        self.n_mid = self.H * self.V
+        self.names = {"q": self.H * 2 * self.D}
+        if self.kv_from is None:
+            self.names.update(k=self.G * 2 * self.D, v=self.G * self.V)
+        self.C = sum(self.names.values())
+
+    def tensor_shapes(self):
+        self._dims()
+        d = {"o": (self.width, self.n_mid)}
+        d.update({k: (self.D,) for k in ("lq1", "lk1", "lq2", "lk2")})
+        for k, n in self.names.items():
+            d.update({k: (n, self.width), k + ".conv": (n, self.K)})
+        return d
+
+    def load(self, get, dtype, dev):
+        self._dims()
+        # one projection for everything that reads the layer input: q | k | v
+        self.w_in = torch.cat([get(k) for k in self.names], 0).to(dev, dtype).contiguous()
+        self.cw = torch.cat([_vec(get(k + ".conv"), dev) for k in self.names], 0).contiguous()
+        lq1, lk1, lq2, lk2 = (get(k).double() for k in ("lq1", "lk1", "lq2", "lk2"))
+        self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
+        self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev, self.rot_scaling)
+        if sm.rope_magnitude(self.rot_scaling) != 1.0:
+            raise ValueError("diff_attention: the convolved input pass has no rotation magnitude")
+        self.wo = get("o").to(dev, dtype).contiguous()
+
+    def cache_spec(self):
+        tail = ("state", {"tail": (self.K - 1, self.C)})
+        return [("paged", self.G * (2 * self.D + self.V)), tail] if self.kv_from is None else [tail]
+
+    def shares_cache_with(self, other) -> bool:
+        """Whether this layer can read the keys and values that ``other`` leaves in its pool."""
+        return (isinstance(other, DiffAttention) and other.kv_from is None
+                and (other.G, other.D, other.V) == (self.G, self.D, self.V)
+                and (other.rot_dims, other.rot_base, other.rot_scaling)
+                == (self.rot_dims, self.rot_base, self.rot_scaling))
+
+    def mix(self, proj, b, cache, layer, out, out_scale=1.0):
+        H, G, D, V = self.H, self.G, self.D, self.V
+        own = self.kv_from is None
+        pool = cache.paged[layer if own else self.kv_from]
+        q = torch.empty(b.R, H * 2 * D, device=proj.device, dtype=proj.dtype)
+        sm.conv_rope_norm_store(proj, H, G, D, V, self.cw, cache.state[layer]["tail"], self.inv_freq, None,
+                                b.pos, b.cache_rows, pool if own else None, self.eps, q, b.ent, b.ent_host,
+                                b.row_ent, b.block_tables, PAGE, maps=2, norm=False)
+        units = b.units(sm.window_rows_per_wave(H // G)) if sm.window_mfma_ok(q, pool, D, V) else None
+        sm.window_attn(q, pool, b.block_tables, b.row_ent, b.pos, None, self.scale, self.win, out, PAGE,
+                       H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale * (1.0 - self.diff),
+                       keep=self.keep, diff=(self.lam, self.eps))
+        return out
+
+
 class RopeLatentAttention(Mixer):
     """Latent attention with a rotated key part (``ops.seqmix.latent_attn``): queries come
     through a normed low-rank latent; every token caches its normed key/value latent c
@@ -789,18 +897,23 @@ class RopeLatentAttention(Mixer):
     A head's score is q_plain . (W_uk c) + q_rot . k_rot; the first term is evaluated in latent
     space, (W_uk^T q_plain) . c, so keys and values are never formed: the cached row [c | k_rot]
     meets the query [W_uk^T q_plain | q_rot], and the attended latent leaves through W_uv.
-    Rotation turns the pairs (2i, 2i+1).  Plain causal softmax (``mask`` optional), one sigmoid
-    gate per head."""
+    Rotation turns the pairs (2i, 2i+1) (``rot.scaling``: optional stretching of long wavelengths).
+    Plain causal softmax (``mask`` optional), one sigmoid gate per head."""
     kind = "rope_latent_attention"
+    QUERY_LATENT = True   # queries through a normed latent, or projected straight from the input
+    HEAD_GATE = True      # one sigmoid gate per head on the way out
 
     def _dims(self):
         s = self.spec
         self.H, self.D, self.V = int(s["heads"]), int(s["dim"]), int(s["vdim"])
-        self.Rd, self.rank, self.qrank = int(s["rot_dim"]), int(s["kv_rank"]), int(s["q_rank"])
+        self.Rd, self.rank, self.qrank = int(s["rot_dim"]), int(s["kv_rank"]), int(s.get("q_rank", 0))
         self.win = int(s["mask"]["size"]) if s.get("mask") else 1 << 30
         self.scale = float(s["scale"]) if "scale" in s else (self.D + self.Rd) ** -0.5
         rot = s.get("rot") or {"dims": self.Rd, "base": 10000.0}
         self.rot_dims, self.rot_base = int(rot["dims"]), float(rot["base"])
+        self.rot_scaling = dict(rot["scaling"]) if rot.get("scaling") else None
+        if self.QUERY_LATENT and self.qrank < 1:
+            raise ValueError("rope_latent_attention: query latent of %d numbers" % self.qrank)
         if self.rot_dims % 2 or self.rot_dims > self.Rd:
             raise ValueError("rope_latent_attention: %d rotated of %d channels" % (self.rot_dims, self.Rd))
         self.n_mid = self.H * self.V
@@ -814,20 +927,27 @@ class RopeLatentAttention(Mixer):
     def tensor_shapes(self):
         self._dims()
         H, D, V, Rd, r, qr, W = self.H, self.D, self.V, self.Rd, self.rank, self.qrank, self.width
-        return {"dq": (qr, W), "dq.norm": (qr,), "uq": (H * (D + Rd), qr), "dkv": (r + Rd, W),
-                "dkv.norm": (r,), "uk": (H * D, r), "uv": (H * V, r), "g": (H, W), "o": (W, H * V)}
+        d = {"dq": (qr, W), "dq.norm": (qr,), "uq": (H * (D + Rd), qr)} if self.QUERY_LATENT else \
+            {"q": (H * (D + Rd), W)}
+        d.update({"dkv": (r + Rd, W), "dkv.norm": (r,), "uk": (H * D, r), "uv": (H * V, r), "o": (W, H * V)})
+        if self.HEAD_GATE:
+            d["g"] = (H, W)
+        return d
 
     def load(self, get, dtype, dev):
         self._dims()
         H, D, V, r = self.H, self.D, self.V, self.rank
-        # one projection for everything that reads the layer input: query latent | key/value
-        # latent | rotated key part | head gates
-        self.w_in = torch.cat([get("dq"), get("dkv"), get("g")], 0).to(dev, dtype).contiguous()
-        self.qnorm, self.cnorm = _vec(get("dq.norm"), dev), _vec(get("dkv.norm"), dev)
-        self.uq = get("uq").to(dev, dtype).contiguous()
+        # one projection for everything that reads the layer input: query latent (or queries) |
+        # key/value latent | rotated key part | head gates
+        names = ["dq" if self.QUERY_LATENT else "q", "dkv"] + (["g"] if self.HEAD_GATE else [])
+        self.w_in = torch.cat([get(k) for k in names], 0).to(dev, dtype).contiguous()
+        self.cnorm = _vec(get("dkv.norm"), dev)
+        if self.QUERY_LATENT:
+            self.qnorm, self.uq = _vec(get("dq.norm"), dev), get("uq").to(dev, dtype).contiguous()
         self.uk = get("uk").to(dev, dtype).view(H, D, r).contiguous()
         self.uvt = get("uv").to(dev, dtype).view(H, V, r).transpose(1, 2).contiguous()
-        self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev)
+        self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev, self.rot_scaling)
+        self.rot_mag = sm.rope_magnitude(self.rot_scaling)
         self.wo = get("o").to(dev, dtype).contiguous()
 
     def cache_spec(self):
@@ -837,26 +957,45 @@ class RopeLatentAttention(Mixer):
         H, D, V, Rd, r, qr = self.H, self.D, self.V, self.Rd, self.rank, self.qrank
         R, dev, dt = b.R, proj.device, proj.dtype
         pool = cache.paged[layer]
-        cq = torch.empty(R, qr, device=dev, dtype=dt)
-        sm.latent_prep(proj, qr, r, Rd, self.qnorm, self.cnorm, self.inv_freq, b.pos, b.cache_rows,
-                       pool, self.eps, cq)
-        q = F.linear(cq, self.uq)                                                  # [R, H*(D+Rd)]
+        if self.QUERY_LATENT:
+            cq = torch.empty(R, qr, device=dev, dtype=dt)
+            sm.latent_prep(proj, qr, r, Rd, self.qnorm, self.cnorm, self.inv_freq, b.pos, b.cache_rows,
+                           pool, self.eps, cq, rm=self.rot_mag)
+            q = F.linear(cq, self.uq)                                              # [R, H*(D+Rd)]
+        else:
+            qr = H * (D + Rd)
+            q = proj[:, :qr]
+            sm.latent_prep(proj[:, qr:], 0, r, Rd, None, self.cnorm, self.inv_freq, b.pos, b.cache_rows,
+                           pool, self.eps, None, rm=self.rot_mag)
         nrot2 = self.rot_dims
         qa = torch.empty(H, R, r + Rd, device=dev, dtype=dt)
-        q3 = q.view(R, H, D + Rd)
+        q3 = q.unflatten(1, (H, D + Rd))
         torch.bmm(q3[:, :, :D].transpose(0, 1), self.uk, out=qa[:, :, :r])
-        sm.rope_rows(q[:, D:], H, D + Rd, self.inv_freq, b.pos, qa[0, :, r:], qa.stride(0))
+        sm.rope_rows(q[:, D:], H, D + Rd, self.inv_freq, b.pos, qa[0, :, r:], qa.stride(0),
+                     rm=self.rot_mag)
         if nrot2 < Rd:
             qa[:, :, r + nrot2:] = q3[:, :, D + nrot2:].transpose(0, 1)
         ol = torch.empty_like(qa)
         units = b.units(sm.latent_rows_per_wave(H)) if sm.latent_mfma_ok(qa, pool) else None
         sm.latent_attn(qa, pool, b.block_tables, b.row_ent, b.pos, None, self.scale, self.win, ol,
                        PAGE, units=units, max_keys=b.max_keys)
+        if not self.HEAD_GATE:
+            torch.bmm(ol[:, :, :r], self.uvt, out=out.unflatten(1, (H, V)).transpose(0, 1))
+            if out_scale != 1.0:
+                out.mul_(out_scale)
+            return out
         o = torch.bmm(ol[:, :, :r], self.uvt)                                      # [H, R, V]
         sm.sigmoid_gate(o, proj[:, qr + r + Rd:], out, H, V, per_head=True)
         if out_scale != 1.0:
             out.mul_(out_scale)
         return out
+
+
+class DirectLatentAttention(RopeLatentAttention):
+    """Latent attention with a rotated key part whose queries are projected straight from the layer
+    input, without a gate."""
+    kind = "direct_latent_attention"
+    QUERY_LATENT = HEAD_GATE = False
 
 
 class MLSTM(Mixer):
@@ -986,6 +1125,51 @@ class HGRN2(Mixer):
         return out
 
 
+class GLA(Mixer):
+    """Gated linear attention (``ops.seqmix.gla_scan``): S <- diag(decay) S + k v^T with a decay per key
+    channel, sigmoid(W_a2 W_a1 h + b)^(1 / tau); a norm over every head's V channels with a weight shared by
+    the heads, a silu gate per channel."""
+    kind = "gla"
+    LOW_RANK = 16
+
+    @staticmethod
+    def resolve_spec(spec, prefix, shapes):
+        if "decay_rank" not in spec and prefix + "a1" in shapes:
+            spec["decay_rank"] = int(tuple(shapes[prefix + "a1"])[0])
+        return spec
+
+    def _dims(self):
+        s = self.spec
+        self.H, self.D, self.V, self.tau = int(s["heads"]), int(s["dim"]), int(s["vdim"]), float(s["tau"])
+        self.ra = int(s.get("decay_rank", self.LOW_RANK))
+        if self.tau <= 0 or self.ra < 1:
+            raise ValueError("gla: tau %g / decay rank %d" % (self.tau, self.ra))
+        self.n_mid = self.H * self.V
+
+    def tensor_shapes(self):
+        self._dims()
+        n, nv, W = self.H * self.D, self.n_mid, self.width
+        return {"q": (n, W), "k": (n, W), "v": (nv, W), "g": (nv, W), "a1": (self.ra, W), "a2": (n, self.ra),
+                "a2.b": (n,), "norm": (self.V,), "o": (W, nv)}
+
+    def load(self, get, dtype, dev):
+        self._dims()
+        # one projection for everything that reads the layer input: q | k | v | gate | a1
+        self.w_in = torch.cat([get(k) for k in ("q", "k", "v", "g", "a1")], 0).to(dev, dtype).contiguous()
+        self.w_a2 = get("a2").to(dev, dtype).contiguous()
+        self.za, self.normw = _vec(get("a2.b"), dev), _vec(get("norm"), dev)
+        self.wo = get("o").to(dev, dtype).contiguous()
+
+    def cache_spec(self):
+        return ("state", {"S": (self.H, self.D, self.V)})
+
+    def mix(self, proj, b, cache, layer, out, out_scale=1.0):
+        sm.gla_scan(proj, 2 * self.H * self.D + 2 * self.n_mid, self.ra, self.w_a2, self.za, 1.0 / self.tau,
+                    self.normw, cache.state[layer]["S"], b.ent, b.ent_host, out, self.H, self.D, self.V,
+                    self.eps, out_scale=out_scale)
+        return out
+
+
 class Parallel(Mixer):
     """Two mixers on the same input: ``left_scale * left + right_scale * right``.  Their input
     projections are one matrix product, and so are their output projections (each branch
@@ -998,9 +1182,9 @@ class Parallel(Mixer):
         self.parts = [(name, MIXERS[spec[name].get("type", kind)](dict(spec[name]), width, eps),
                        float(spec.get(name + "_scale", 1.0))) for name, kind in self.BRANCHES]
 
-    @staticmethod
-    def resolve_spec(spec, prefix, shapes):
-        for name, kind in Parallel.BRANCHES:
+    @classmethod
+    def resolve_spec(cls, spec, prefix, shapes):
+        for name, kind in cls.BRANCHES:
             sub = dict(spec[name])
             spec[name] = MIXERS[sub.get("type", kind)].resolve_spec(sub, prefix + name + ".", shapes)
         return spec
@@ -1031,9 +1215,16 @@ class Parallel(Mixer):
         return out
 
 
+class ParallelGLA(Parallel):
+    """Attention beside gated linear attention."""
+    kind = "parallel_gla"
+    BRANCHES = (("left", "attention"), ("right", "gla"))
+
+
 MIXERS = {c.kind: c for c in (GeneralDelta, Mamba2, LatentAttention, WindowAttention, GatedDelta,
                               HGRN2, Parallel, Attention, MLSTM, BiasedAttention, RopeLatentAttention,
-                              ConvAttention, Mamba1, Lightning)}
+                              ConvAttention, Mamba1, Lightning, DiffAttention, DirectLatentAttention, GLA,
+                              ParallelGLA)}
 
 
 class DenseFF:
@@ -1228,6 +1419,8 @@ class TopMoEFF:
     same form runs for every token; its products ride on the layer's input and output
     products."""
 
+    BIAS = True   # the router has a bias
+
     def __init__(self, spec: dict, width: int):
         self.spec, self.width = spec, width
         r = spec["router"]
@@ -1238,7 +1431,9 @@ class TopMoEFF:
             raise ValueError("moe: %d experts, %d chosen" % (self.E, self.top))
 
     def tensor_shapes(self):
-        d = {"router": (self.E, self.width), "router.b": (self.E,)}
+        d = {"router": (self.E, self.width)}
+        if self.BIAS:
+            d["router.b"] = (self.E,)
         for e in range(self.E):
             d.update({"e%d.gate" % e: (self.F, self.width), "e%d.up" % e: (self.F, self.width),
                       "e%d.down" % e: (self.width, self.F)})
@@ -1248,7 +1443,8 @@ class TopMoEFF:
         return d
 
     def load(self, get, dtype, dev):
-        self.wr, self.br = get("router").to(dev).float().contiguous(), _vec(get("router.b"), dev)
+        self.wr = get("router").to(dev).float().contiguous()
+        self.br = _vec(get("router.b"), dev) if self.BIAS else None
         gate = torch.stack([get("e%d.gate" % e) for e in range(self.E)])
         up = torch.stack([get("e%d.up" % e) for e in range(self.E)])
         # widths that are multiples of 16: gate and up rows interleaved, so that the first
@@ -1262,6 +1458,10 @@ class TopMoEFF:
             self.w_in = torch.cat([get("shared.gate"), get("shared.up")], 0).to(dev, dtype).contiguous()
             self.w_out = get("shared.down").to(dev, dtype).contiguous()
 
+    def route(self, h, ids, wts, cnt, rows, cleared: bool):
+        sm.group_route(h, self.wr, self.top, 1, 1, ids, wts, cnt, rows, score="top_softmax", bias=self.br,
+                       cleared=cleared)
+
     def routed(self, h, cnt=None):
         """(y [R * top, width], wts [R, top]): the chosen experts' outputs and their weights,
         to be summed by whoever adds them to the residual.  cnt: cleared int32 counts [E] (a
@@ -1273,8 +1473,7 @@ class TopMoEFF:
         if cnt is None:
             cnt = torch.empty(self.E, device=dev, dtype=torch.int32)
         rows = torch.empty(self.E, R * top, device=dev, dtype=torch.int32)
-        sm.group_route(h, self.wr, top, 1, 1, ids, wts, cnt, rows, score="top_softmax", bias=self.br,
-                       cleared=cleared)
+        self.route(h, ids, wts, cnt, rows, cleared)
         act = torch.empty(R * top, self.F, device=dev, dtype=h.dtype)
         if self.fused:
             sm.expert_gemm(h, top, self.w_gu, cnt, rows, act, R * top, silu_glu=True)
@@ -1306,25 +1505,79 @@ class TopMoEFF:
         return y
 
 
+class GroupMoEFF(TopMoEFF):
+    """The same experts behind a softmax router with group-limited choice: s = softmax(W_r h) over all
+    experts; only experts of the ``groups.keep`` groups of neighbours with the largest best score can
+    be chosen; the weights are the winners' s divided by their sum, times ``router.scale``."""
+    BIAS = False
+
+    def __init__(self, spec: dict, width: int):
+        super().__init__(spec, width)
+        g = spec["router"].get("groups") or {}
+        self.groups = int(g.get("count", 1))
+        self.keep, self.wscale = int(g.get("keep", self.groups)), float(spec["router"].get("scale", 1.0))
+        if self.groups < 1 or self.E % self.groups or not 1 <= self.keep <= self.groups \
+                or self.top > self.keep * (self.E // self.groups):
+            raise ValueError("moe: %d experts in %d groups, %d kept, %d chosen"
+                             % (self.E, self.groups, self.keep, self.top))
+
+    def route(self, h, ids, wts, cnt, rows, cleared: bool):
+        sm.group_route(h, self.wr, self.top, self.groups, self.keep, ids, wts, cnt, rows, score="softmax",
+                       group_score="max", renorm=True, scale=self.wscale, cleared=cleared)
+
+
 FEEDFORWARDS = {"dense": DenseFF, "moe": MoEFF, "dense_gelu": GeluFF, "moe_softmax": SoftmaxMoEFF,
-                "moe_top": TopMoEFF}
+                "moe_top": TopMoEFF, "moe_group": GroupMoEFF}
 
 
 # ---------------------------------------------------------------------------- weights
+class DynamicTanh:
+    """Norm without statistics: tanh(alpha x) * w + b, alpha one number."""
+
+    @staticmethod
+    def tensor_shapes(name: str, width: int) -> dict:
+        return {name: (width,), name + ".b": (width,), name + ".alpha": ()}
+
+    def __init__(self, sd, name: str, dev):
+        self.args = (float(sd[name + ".alpha"].float()), _vec(sd[name], dev), _vec(sd[name + ".b"], dev))
+
+
+class HyperConnection:
+    """Coefficients of a sublayer on parallel residual streams: what it reads (``read``), how the
+    streams exchange (``mix`` [from, to]) and where its result goes (``out``)."""
+
+    @staticmethod
+    def tensor_shapes(name: str, streams: int) -> dict:
+        return {name + ".in": (streams,), name + ".mix": (streams, streams), name + ".out": (streams,)}
+
+    def __init__(self, sd, name: str, dev):
+        self.read, self.mix, self.out = (_vec(sd[name + k], dev) for k in (".in", ".mix", ".out"))
+
+
 class HybridLayer:
     def __init__(self, spec: LayerSpec, cfg: HybridConfig):
         self.block = cfg.traits.block
-        self.norm_offset = cfg.traits.norm_offset
+        self.norm_offset, self.streams = cfg.traits.norm_offset, cfg.streams
         self.mixer = MIXERS[cfg.traits.mixer_key(spec.kind)](spec.mixer, cfg.width, cfg.eps)
         self.ff = FEEDFORWARDS[cfg.traits.ff_key(spec.mlp.get("kind", "dense"))](spec.mlp, cfg.width) \
             if spec.mlp is not None else None
         # parallel: the layer's input and output products (mixer and feed-forward together)
         self.w_in_all = self.w_out_all = None
         self.norm1 = self.norm1b = self.ls1 = self.norm2 = self.norm2b = self.ls2 = None
+        # streams: the sublayers' connections to the residual streams
+        self.hc1 = self.hc2 = None
         # gated_post: the gates' projections ride on the sublayers' input products
         self.w_in1 = self.w_in2 = self.rg1b = self.rg2b = None
 
     def tensor_shapes(self, W):
+        if self.block == "streams":
+            d = {}
+            for q, part, name in ((1, self.mixer, "mix."), (2, self.ff, "mlp.")):
+                if part is not None:
+                    d.update(DynamicTanh.tensor_shapes("norm%d" % q, W))
+                    d.update(HyperConnection.tensor_shapes("hc%d" % q, self.streams))
+                    d.update({name + k: s for k, s in part.tensor_shapes().items()})
+            return d
         if self.block == "parallel2":
             d = {"norm1": ()}
             d.update({"mix." + k: s for k, s in self.mixer.tensor_shapes().items()})
@@ -1359,6 +1612,11 @@ class HybridLayer:
         self.mixer.load(lambda k: sd[p + "mix." + k], dtype, dev)
         if self.ff is not None:
             self.ff.load(lambda k: sd[p + "mlp." + k], dtype, dev)
+        if self.block == "streams":
+            self.norm1, self.hc1 = DynamicTanh(sd, p + "norm1", dev), HyperConnection(sd, p + "hc1", dev)
+            if self.ff is not None:
+                self.norm2, self.hc2 = DynamicTanh(sd, p + "norm2", dev), HyperConnection(sd, p + "hc2", dev)
+            return
         if self.block == "parallel2":
             # the mixer and the feed-forward read the same rows through norms of their own, so
             # each has its input product; their output products are one
@@ -1409,6 +1667,8 @@ def tensor_shapes(cfg: HybridConfig) -> dict:
     """name -> shape of every tensor of a checkpoint of this config."""
     W = cfg.width
     d = {"embed": (cfg.vocab, W), "final.norm": () if cfg.traits.scalar_norms else (W,)}
+    if cfg.traits.block == "streams":
+        d.update(DynamicTanh.tensor_shapes("final.norm", W))
     if not cfg.traits.tied_head:
         d["head"] = (cfg.vocab, W)
     if cfg.traits.positions:
@@ -1436,7 +1696,8 @@ class HybridWeights:
                 raise ValueError("tensor %r has shape %s, the config gives %s" % (k, tuple(sd[k].shape), s))
         self.embed = sd["embed"].to(dev, dtype).contiguous()
         self.pos = sd["pos"].to(dev, dtype).contiguous() if cfg.traits.positions else None
-        self.final_norm = (_vec(sd["final.norm"], dev) + cfg.traits.norm_offset).expand(cfg.width).contiguous() \
+        self.final_norm = DynamicTanh(sd, "final.norm", dev) if cfg.traits.block == "streams" else \
+            (_vec(sd["final.norm"], dev) + cfg.traits.norm_offset).expand(cfg.width).contiguous() \
             if cfg.traits.scalar_norms else (_vec(sd["final.norm"], dev) + cfg.traits.norm_offset).contiguous()
         self.head = self.embed if cfg.traits.tied_head else sd["head"].to(dev, dtype).contiguous()
         self.loop_step = _vec(sd["loop.step"], dev) if cfg.loop else None
@@ -1476,7 +1737,18 @@ def random_state_dict(cfg: HybridConfig, seed: int = 0) -> dict:
     for k, s in shapes.items():
         s = tuple(s) or (1,)   # a single number is drawn as one and stored without a shape
         leaf = k.split(".", 1)[1] if k.startswith("l") and "." in k else k
-        if len(s) == 2 and not leaf.endswith("conv"):
+        if leaf.startswith("hc"):
+            t = torch.randn(*s, generator=g) * 0.2 + (torch.eye(s[0]) if leaf.endswith("mix") else
+                                                      1.0 if leaf.endswith("out") else 1.0 / s[0])
+        elif leaf.endswith(".alpha"):
+            t = 0.5 + 0.2 * torch.rand(*s, generator=g)
+        elif leaf in ("norm1.b", "norm2.b", "final.norm.b"):
+            t = torch.randn(*s, generator=g) * 0.2
+        elif leaf.endswith(("mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2")):
+            t = torch.randn(*s, generator=g) * 0.3
+        elif leaf.endswith("a2.b"):
+            t = torch.randn(*s, generator=g) * 1.5 + 1.5
+        elif len(s) == 2 and not leaf.endswith("conv"):
             t = torch.randn(*s, generator=g) / (s[1] ** 0.5 if k not in ("embed", "pos") else 1.0)
         elif leaf.endswith("conv"):
             t = torch.randn(*s, generator=g) * 0.5
@@ -1541,6 +1813,8 @@ class HybridModel:
             return self._forward_parallel2(b, layer_out)
         if cfg.traits.block == "post":
             return self._forward_post(b, layer_out)
+        if cfg.traits.block == "streams":
+            return self._forward_streams(b, layer_out)
         x = torch.empty(b.R, cfg.width, device=self.device, dtype=torch.float32)
         sm.embed_pos(w.embed, w.pos, b.ids, b.pos, x)
         h = torch.empty(b.R, cfg.width, device=self.device, dtype=self.dtype)
@@ -1566,11 +1840,60 @@ class HybridModel:
         cfg, w = self.cfg, self.w
         hn = torch.empty(b.n_out, cfg.width, device=self.device, dtype=self.dtype)
         sm.rmsnorm(x, w.final_norm, cfg.eps, hn, parts=cfg.norm_groups, in_rows=b.out_rows)
+        return self._head(hn)
+
+    def _head(self, hn):
+        cfg, w = self.cfg, self.w
         y = F.linear(hn, w.head)
         if not cfg.logit_softcap and cfg.logit_scale == 1.0:
             return y.float()
         return sm.softcap(y, cfg.logit_softcap, torch.empty(y.shape, device=y.device, dtype=torch.float32),
                           scale=cfg.logit_scale)
+
+    def _forward_streams(self, b: StepBatch, layer_out=None):
+        """x_t <- sum_s M[s, t] x_s + c_t f(N(sum_s a_s x_s)) per sublayer, N a dynamic tanh: one pointwise
+        pass updates all streams (the routed experts' sum included) and forms the next sublayer's
+        input; the last one reads only the wanted rows and goes straight to the final norm."""
+        cfg, w = self.cfg, self.w
+        R, W, dev = b.R, cfg.width, self.device
+        x = torch.empty(R, cfg.streams, W, device=dev, dtype=torch.float32)
+        h = torch.empty(R, W, device=dev, dtype=self.dtype)
+        moe = [hasattr(L.ff, "fill_routed") for L in w.layers]
+        # the experts' slot counts of all layers, cleared by one fill
+        cnts = torch.zeros(sum(moe), max([L.ff.E for L, m in zip(w.layers, moe) if m] or [1]), device=dev,
+                           dtype=torch.int32) if any(moe) else None
+        subs = [(i, q) for i, L in enumerate(w.layers) for q in (1, 2) if q == 1 or L.ff is not None]
+        side = lambda i, q: (getattr(w.layers[i], "hc%d" % q), getattr(w.layers[i], "norm%d" % q))
+        hc, norm = side(*subs[0])
+        sm.stream_mix(x, embed=(w.embed, b.ids, cfg.embed_scale), read=hc.read, dyt=norm.args, h=h)
+        hn = torch.empty(b.n_out, W, device=dev, dtype=self.dtype) if b.n_out else None
+        for k, (i, q) in enumerate(subs):
+            L, (hc, _n) = w.layers[i], side(i, q)
+            y = routed = None
+            if q == 1:
+                y = L.mixer.forward(h, b, self.cache, i)
+            elif moe[i]:
+                mid = proj = None
+                if L.ff.n_mid:
+                    proj = F.linear(h, L.ff.w_in)
+                    mid = torch.empty(R, L.ff.n_mid, device=dev, dtype=self.dtype)
+                routed = L.ff.fill_routed(proj, h, mid, cnts[sum(moe[:i]), :L.ff.E])
+                y = F.linear(mid, L.ff.w_out) if mid is not None else None
+            else:
+                y = L.ff.forward(h)
+            if k + 1 < len(subs):
+                nhc, nnorm = side(*subs[k + 1])
+                sm.stream_mix(x, y, None, routed, hc.mix, hc.out, nhc.read, nnorm.args, h)
+            elif layer_out is not None:
+                sm.stream_mix(x, y, None, routed, hc.mix, hc.out)
+                if b.n_out:
+                    sm.stream_mix(x, dyt=w.final_norm.args, h=hn, rows=b.out_rows, write=False)
+            elif b.n_out:
+                sm.stream_mix(x, y, None, routed, hc.mix, hc.out, None, w.final_norm.args, hn,
+                              rows=b.out_rows, write=False)
+            if layer_out is not None and (k + 1 == len(subs) or subs[k + 1][0] != i):
+                layer_out.append(x.sum(1))
+        return self._head(hn) if b.n_out else None
 
     def _forward_parallel2(self, b: StepBatch, layer_out=None):
         """x <- x + mixer(N(x) g1) + ff(N(x) g2) over the layer runs of the config (a stretch of

@@ -70,7 +70,7 @@ _SIGS = {
                               c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_lightning_chunked": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
                                  c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
-    "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
+    "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
                                     c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -104,9 +104,9 @@ _SIGS = {
                          c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
     "p2p_sm_latent_prep": [c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p,
                            c_int, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int,
-                           c_int, c_void_p],
+                           c_float, c_int, c_void_p],
     "p2p_sm_rope_rows": [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p,
-                         c_void_p, c_long, c_long, c_int, c_int, c_void_p],
+                         c_void_p, c_long, c_long, c_int, c_float, c_int, c_void_p],
     "p2p_sm_qtemp_kv_store": [c_void_p, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p,
                               c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
     "p2p_sm_mlstm_scan": [c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
@@ -118,16 +118,25 @@ _SIGS = {
                           c_int, c_void_p],
     "p2p_sm_qk_norm_rope_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
                                   c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float,
-                                  c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                  c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p],
+    "p2p_sm_diff_combine": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float,
+                            c_float, c_int, c_void_p],
+    "p2p_sm_stream_mix": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int,
+                          c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                          c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int,
+                          c_int, c_void_p],
+    "p2p_sm_gla_scan": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
+                        c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
+                        c_void_p],
     "p2p_sm_window_attn": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                            c_void_p, c_float, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
                            c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int,
-                           c_int, c_void_p, c_int, c_int, c_void_p],
+                           c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_window_attn_mfma": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                                 c_void_p, c_int, c_void_p, c_float, c_int, c_void_p, c_int, c_int,
                                 c_int, c_int, c_int, c_int, c_int, c_void_p, c_float, c_float,
                                 c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int,
-                                c_void_p],
+                                c_int, c_int, c_float, c_float, c_void_p],
     "p2p_sm_hgrn2_scan": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                           c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
                           c_void_p],
@@ -145,7 +154,7 @@ _SIGS = {
                                 c_int, c_void_p],
     "p2p_sm_group_route": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                            c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                           c_void_p, c_int, c_void_p],
+                           c_void_p, c_int, c_float, c_int, c_void_p],
     "p2p_sm_expert_gemm": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                            c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
                            c_void_p],
@@ -438,6 +447,94 @@ def add_norm2(x, a=None, b=None, rows=None, vec=None, eps: float = 0.0, w1=None,
                                 _lib.ptr(out2), ld2, _lib.ptr(cy), ldcy, _lib.ptr(cw), top,
                                 _f32(act) if act is not None else 1, _st(x)),
          "add_norm2")
+    return x
+
+
+MAX_STREAMS = 8
+
+
+def stream_mix(x, a=None, b=None, routed=None, mix=None, out=None, read=None, dyt=None, h=None, rows=None,
+               write: bool = True, embed=None):
+    """Residual of parallel streams, x fp32 [R, n streams, width].  In one pass:
+      * embed = (table, ids, scale): every stream becomes table[ids[r]] * scale (a step's start);
+      * or with mix (fp32 [streams, streams], indexed [from, to]) and out (fp32 [streams]):
+        x_t <- sum_s mix[s, t] x_s + out[t] y, all streams from the old ones, with
+        y = a + b + routed as in ``add_norm2`` (each optional), summed in fp32;
+      * h (activation type) receives sum_s read[s] x_s of the updated streams (read None: their sum),
+        with dyt = (alpha, w, bias) as tanh(alpha * .) * w + bias (a dynamic tanh norm).
+    rows (int32): only these rows of x are taken, output row i is x row rows[i]; such a pass does
+    not store the streams (write=False)."""
+    R, NS, n = x.shape
+    if embed is not None and mix is not None:
+        raise ValueError("stream_mix: a step's start has nothing to mix")
+    if rows is not None and write:
+        raise ValueError("stream_mix: a pass over chosen rows does not store them")
+    Ro = R if rows is None else rows.numel()
+    if not x.is_cuda:
+        xs = x if rows is None else x[rows.long()]
+        sel = slice(0, R) if rows is None else rows.long()
+        if embed is not None:
+            xs = (embed[0][embed[1][sel].long()].float() * embed[2])[:, None].expand(Ro, NS, n).clone()
+        elif mix is not None:
+            y = torch.zeros(Ro, n)
+            for t in (a, b):
+                if t is not None:
+                    y = y + t[sel].float()
+            if routed is not None:
+                ry, rw = routed
+                y = y + (ry[:R * rw.shape[1]].float().view(R, rw.shape[1], n)[sel] * rw[sel][:, :, None]).sum(1)
+            xs = torch.einsum("rsn,st->rtn", xs, mix) + out[None, :, None] * y[:, None]
+        if write:
+            x.copy_(xs)
+        if h is not None:
+            u = xs.sum(1) if read is None else torch.einsum("rsn,s->rn", xs, read)
+            if dyt is not None:
+                u = torch.tanh(dyt[0] * u) * dyt[1] + dyt[2]
+            h[:Ro] = u.to(h.dtype)
+        return x
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    if NS > MAX_STREAMS:
+        raise ValueError("stream_mix: %d streams > %d" % (NS, MAX_STREAMS))
+    if rows is not None:
+        assert rows.dtype == torch.int32 and rows.is_contiguous()
+    act, ld = None, {}
+    for nm, t in (("a", a), ("b", b), ("h", h)):
+        ld[nm] = 0
+        if t is not None:
+            _rows2d(t, nm)
+            assert t.shape[1] == n and t.shape[0] >= (Ro if nm == "h" else R), nm
+            assert act is None or t.dtype == act.dtype, nm
+            act, ld[nm] = t, t.stride(0)
+    cy = cw = None
+    ldcy = top = 0
+    if routed is not None:
+        cy, cw = routed
+        top = cw.shape[1]
+        _rows2d(cy, "routed y")
+        assert cy.shape[1] == n and cy.shape[0] >= R * top and (act is None or cy.dtype == act.dtype)
+        assert cw.dtype == torch.float32 and cw.is_contiguous() and cw.shape[0] >= R
+        act, ldcy = cy, cy.stride(0)
+    table = ids = None
+    scale = 1.0
+    if embed is not None:
+        table, ids, scale = embed
+        assert table.is_contiguous() and table.shape[1] == n and (act is None or table.dtype == act.dtype)
+        assert ids.dtype == torch.int32 and ids.numel() >= R
+        act = table
+    if mix is not None:
+        _vec(mix.view(-1), NS * NS, "mix")
+        _vec(out, NS, "out")
+    if read is not None:
+        _vec(read, NS, "read")
+    alpha, w, bias = dyt if dyt is not None else (0.0, None, None)
+    if w is not None:
+        _vec(w, n, "dyt weight")
+        _vec(bias, n, "dyt bias")
+    _chk(lib().p2p_sm_stream_mix(
+        x.data_ptr(), Ro, NS, n, _lib.ptr(rows), _lib.ptr(a), ld["a"], _lib.ptr(b), ld["b"], _lib.ptr(cy),
+        ldcy, _lib.ptr(cw), top, _lib.ptr(mix), _lib.ptr(out if mix is not None else None),
+        _lib.ptr(read), _lib.ptr(w), _lib.ptr(bias), alpha, _lib.ptr(h), ld["h"], _lib.ptr(table),
+        _lib.ptr(ids), scale, 1 if write else 0, _f32(act) if act is not None else 1, _st(x)), "stream_mix")
     return x
 
 
@@ -1004,10 +1101,25 @@ def rope_inv_freq(base: float, dims: int, device, scaling: dict | None = None) -
 
     scaling = {factor, low, high, original} stretches the long wavelengths: with l = 2 pi / f,
     f stays where l < original / high, becomes f / factor where l > original / low, and in
-    between is (1 - s) f / factor + s f with s = (original / l - low) / (high - low)."""
+    between is (1 - s) f / factor + s f with s = (original / l - low) / (high - low).
+
+    scaling = {factor, original, fast, slow} (YaRN): pair i turns r_i times over ``original``
+    positions, and i(r) is the (fractional) pair that turns r times; pairs up to floor(i(fast)) keep
+    f, pairs from ceil(i(slow)) on turn at f / factor, linear in i between them.  The rotation
+    itself is then scaled by ``rope_magnitude``."""
     i = torch.arange(dims // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
-    if scaling:
+    if scaling and "fast" in scaling:
+        fac, orig = float(scaling["factor"]), float(scaling["original"])
+
+        def pair(turns):
+            return dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+        lo = max(math.floor(pair(float(scaling["fast"]))), 0)
+        hi = min(math.ceil(pair(float(scaling["slow"]))), dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+        f = f / fac * ramp + f * (1.0 - ramp)
+    elif scaling:
         fac, lo, hi = float(scaling["factor"]), float(scaling["low"]), float(scaling["high"])
         orig = float(scaling["original"])
         wl = 2.0 * math.pi / f
@@ -1017,11 +1129,16 @@ def rope_inv_freq(base: float, dims: int, device, scaling: dict | None = None) -
     return f.float().to(device)
 
 
-def rope_rows(src, heads: int, src_hs: int, inv_freq, pos, dst, dst_hs: int, out_rows=None):
+def rope_magnitude(scaling: dict | None) -> float:
+    """Factor on cos and sin that goes with YaRN's frequencies: 0.1 ln(factor) + 1."""
+    return 0.1 * math.log(float(scaling["factor"])) + 1.0 if scaling and "fast" in scaling else 1.0
+
+
+def rope_rows(src, heads: int, src_hs: int, inv_freq, pos, dst, dst_hs: int, out_rows=None, rm: float = 1.0):
     """Rotary positions on a stretch of channels: for every row r and head h < heads the
     pairs (2i, 2i+1), i < len(inv_freq), of src[r, h*src_hs : ...] are turned by the angle
-    pos[r] * inv_freq[i], (a, b) -> (a cos - b sin, b cos + a sin) in fp32, and written to
-    dst[o(r), h*dst_hs : ...]; o(r) = out_rows[r] (a scatter, e.g. into a paged pool) or r.
+    pos[r] * inv_freq[i], (a, b) -> (a cos - b sin, b cos + a sin) in fp32 (cos and sin times rm), and
+    written to dst[o(r), h*dst_hs : ...]; o(r) = out_rows[r] (a scatter, e.g. into a paged pool) or r.
     src and dst are 2-d views that start at the first rotated channel of head 0 (last stride
     1; a head may lie anywhere from there, also beyond the view's own width)."""
     R = src.shape[0]
@@ -1030,7 +1147,7 @@ def rope_rows(src, heads: int, src_hs: int, inv_freq, pos, dst, dst_hs: int, out
         return dst
     if not src.is_cuda:
         ang = pos[:R].float()[:, None] * inv_freq[None, :]
-        c, sn = torch.cos(ang), torch.sin(ang)
+        c, sn = torch.cos(ang) * rm, torch.sin(ang) * rm
         ro = torch.arange(R) if out_rows is None else out_rows[:R].long()
         sv = torch.as_strided(src, (R, heads, 2 * nrot), (src.stride(0), src_hs, 1), src.storage_offset())
         dv = torch.as_strided(dst, (dst.shape[0], heads, 2 * nrot), (dst.stride(0), dst_hs, 1),
@@ -1046,44 +1163,49 @@ def rope_rows(src, heads: int, src_hs: int, inv_freq, pos, dst, dst_hs: int, out
     assert pos.numel() >= R
     _chk(lib().p2p_sm_rope_rows(src.data_ptr(), src.stride(0), heads, src_hs, inv_freq.data_ptr(),
                                 nrot, pos.data_ptr(), _lib.ptr(out_rows), dst.data_ptr(),
-                                dst.stride(0), dst_hs, R, _f32(src), _st(src)), "rope_rows")
+                                dst.stride(0), dst_hs, R, rm, _f32(src), _st(src)), "rope_rows")
     return dst
 
 
 def latent_prep(proj, nq: int, nc: int, nr: int, qw, cw, inv_freq, pos, cache_rows, pool, eps: float,
-                cq_out):
+                cq_out, rm: float = 1.0):
     """Input pass of latent attention with low-rank queries.  proj = [query latent (nq) |
     key/value latent (nc) | key part (nr)] per row: both latents are RMS-normalised by
     themselves and weighted (qw [nq], cw [nc]); the pairs (2i, 2i+1), i < len(inv_freq), of the
     key part are turned by pos * inv_freq[i] (its other channels pass unchanged).  The query
     latent goes to cq_out [R, nq], the key/value latent and the key part to the rows
-    ``cache_rows`` of the paged pool ([tokens, nc + nr]).  Norms, angles, rotation: fp32."""
-    R = cq_out.shape[0]
+    ``cache_rows`` of the paged pool ([tokens, nc + nr]).  cos and sin are taken times rm.  Without a
+    query latent nq is 0 and qw and cq_out are None.  Norms, angles, rotation: fp32."""
+    R = cq_out.shape[0] if nq else proj.shape[0]
     nrot = inv_freq.numel()
     if not proj.is_cuda:
         rows = cache_rows[:R].long()
-        cq_out[:R] = (_rms(proj[:R, :nq].float(), eps) * qw).to(cq_out.dtype)
+        if nq:
+            cq_out[:R] = (_rms(proj[:R, :nq].float(), eps) * qw).to(cq_out.dtype)
         pool[rows, :nc] = (_rms(proj[:R, nq:nq + nc].float(), eps) * cw).to(pool.dtype)
         k = proj[:R, nq + nc:nq + nc + nr].float().clone()
         ang = pos[:R].float()[:, None] * inv_freq[None, :]
-        c, sn = torch.cos(ang), torch.sin(ang)
+        c, sn = torch.cos(ang) * rm, torch.sin(ang) * rm
         a, b = k[:, 0:2 * nrot:2].clone(), k[:, 1:2 * nrot:2].clone()
         k[:, 0:2 * nrot:2] = a * c - b * sn
         k[:, 1:2 * nrot:2] = b * c + a * sn
         pool[rows, nc:] = k.to(pool.dtype)
         return cq_out
     _rows2d(proj, "proj")
-    _rows2d(cq_out, "cq_out")
-    assert proj.shape[1] >= nq + nc + nr and cq_out.shape[1] == nq and cq_out.dtype == proj.dtype
+    assert proj.shape[1] >= nq + nc + nr
+    if nq:
+        _rows2d(cq_out, "cq_out")
+        assert cq_out.shape[1] == nq and cq_out.dtype == proj.dtype
+        _vec(qw, nq, "qw")
     assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == nc + nr and pool.dtype == proj.dtype
-    _vec(qw, nq, "qw")
     _vec(cw, nc, "cw")
     assert inv_freq.dtype == torch.float32 and inv_freq.is_contiguous() and 2 * nrot <= nr
     assert pos.dtype == torch.int32 and cache_rows.dtype == torch.int32
-    _chk(lib().p2p_sm_latent_prep(proj.data_ptr(), proj.stride(0), nq, nc, nr, qw.data_ptr(),
+    _chk(lib().p2p_sm_latent_prep(proj.data_ptr(), proj.stride(0), nq, nc, nr, _lib.ptr(qw if nq else None),
                                   cw.data_ptr(), inv_freq.data_ptr(), nrot, pos.data_ptr(),
-                                  cache_rows.data_ptr(), pool.data_ptr(), eps, cq_out.data_ptr(),
-                                  cq_out.stride(0), R, _f32(proj), _st(proj)), "latent_prep")
+                                  cache_rows.data_ptr(), pool.data_ptr(), eps,
+                                  _lib.ptr(cq_out if nq else None), cq_out.stride(0) if nq else 0, R, rm,
+                                  _f32(proj), _st(proj)), "latent_prep")
     return cq_out
 
 
@@ -1114,12 +1236,14 @@ def qtemp_kv_store(proj, nq: int, nkv: int, coef: float, every: int, pos, cache_
 
 
 def qk_norm_rope_store(proj, H: int, G: int, D: int, V: int, qw, kw, inv_freq, pos, cache_rows,
-                       pool, eps: float, q_out, per_head: bool = False, half: bool = False):
+                       pool, eps: float, q_out, per_head: bool = False, half: bool = False,
+                       rm: float = 1.0):
     """Prepares attention inputs from one projection buffer proj = [q (H*D) | k (G*D) | v (G*V)]:
     q and k are RMS-normalised and weighted -- one mean square per row (heads not separated)
     and weights qw [H*D] / kw [G*D], or with ``per_head`` one mean square per head and weights
     of D channels shared by the heads -- then nrot = len(inv_freq) channel pairs of every head,
-    (2i, 2i+1) or with ``half`` (i, i + nrot), are rotated by pos * inv_freq[i].
+    (2i, 2i+1) or with ``half`` (i, i + nrot), are rotated by pos * inv_freq[i]
+    (cos and sin times rm).
     q goes to q_out [R, H*D]; k | v go to the paged pool rows ``cache_rows`` ([tokens,
     G*D + G*V]).  pool None: the layer reads another layer's keys and values, proj holds only
     q and only q is prepared.  Norm, angles and the rotation are fp32."""
@@ -1128,7 +1252,7 @@ def qk_norm_rope_store(proj, H: int, G: int, D: int, V: int, qw, kw, inv_freq, p
     nrot = inv_freq.numel()
     if not proj.is_cuda:
         ang = (pos[:R].float()[:, None] * inv_freq[None, :])
-        c, s = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+        c, s = torch.cos(ang)[:, None, :] * rm, torch.sin(ang)[:, None, :] * rm
         ia = torch.arange(nrot) if half else torch.arange(0, 2 * nrot, 2)
         ib = ia + nrot if half else ia + 1
 
@@ -1167,7 +1291,7 @@ def qk_norm_rope_store(proj, H: int, G: int, D: int, V: int, qw, kw, inv_freq, p
                                          inv_freq.data_ptr(), nrot, pos.data_ptr(),
                                          cache_rows.data_ptr(), _lib.ptr(pool), eps,
                                          q_out.data_ptr(), q_out.stride(0), R,
-                                         1 if per_head else 0, 1 if half else 0, _f32(proj),
+                                         1 if per_head else 0, 1 if half else 0, rm, _f32(proj),
                                          _st(proj)), "qk_norm_rope_store")
     return q_out
 
@@ -1179,7 +1303,8 @@ def blocks_per_page(page: int, every: int) -> int:
 
 def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_freq, temp, pos,
                          cache_rows, pool, eps: float, q_out, ent, ent_host, row_ent,
-                         block_tables, page: int, blk=None, every: int = 0):
+                         block_tables, page: int, blk=None, every: int = 0, maps: int = 1,
+                         norm: bool = True):
     """Prepares attention inputs from one projection buffer proj = [q (H*D) | k (G*D) | v (G*V) | ..]:
     every channel goes through a causal convolution over time (cw fp32 [C, K], column K-1 the newest
     input, no bias; tail fp32 [slots, K-1, C] the projections before each slot's next token, moved
@@ -1188,9 +1313,14 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
     by temp[h] (fp32 [H] or None).  q goes to q_out [R, H*D], k | v to the rows ``cache_rows`` of the
     paged pool.  All of it fp32.
     blk: a pool of blocks of ``every`` tokens ([pages * blocks_per_page, G*(D+V)]); the blocks that
-    this step's tokens complete get the mean of their tokens' rows of ``pool``."""
+    this step's tokens complete get the mean of their tokens' rows of ``pool``.
+    maps = 2 (differential attention): every q and k head has two parts of D channels, so there are
+    2 H and 2 G of them beside the G value heads.  norm False: q and k heads are not divided by
+    their root mean square.  pool None: the layer reads another layer's keys and values, proj (and
+    cw, tail) hold only q and only q is prepared."""
     R = q_out.shape[0]
-    nq, nk, nv = H * D, G * D, G * V
+    HQ, GK, GV = H * maps, G * maps if pool is not None else 0, G if pool is not None else 0
+    nq, nk, nv = HQ * D, GK * D, GV * V
     C, K = nq + nk + nv, cw.shape[1]
     nrot = inv_freq.numel()
     sb = blocks_per_page(page, every) if blk is not None else 0
@@ -1209,14 +1339,16 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
             u, w = t[:, :, :nrot].clone(), t[:, :, nrot:2 * nrot].clone()
             t[:, :, :nrot] = u * c - w * sn
             t[:, :, nrot:2 * nrot] = w * c + u * sn
-            return _rms(t, eps)
+            return _rms(t, eps) if norm else t
 
-        q = prep(y[:, :nq], H)
+        q = prep(y[:, :nq], HQ)
         if temp is not None:
             q = q * temp[:, None]
         q_out[:R] = q.reshape(R, nq).to(q_out.dtype)
+        if pool is None:
+            return q_out
         rows = cache_rows[:R].long()
-        pool[rows, :nk] = prep(y[:, nq:nq + nk], G).reshape(R, nk).to(pool.dtype)
+        pool[rows, :nk] = prep(y[:, nq:nq + nk], GK).reshape(R, nk).to(pool.dtype)
         pool[rows, nk:] = y[:, nq + nk:].to(pool.dtype)
         if blk is not None:
             bt = block_tables.long()
@@ -1230,7 +1362,9 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
     _rows2d(proj, "proj")
     _rows2d(q_out, "q_out")
     assert proj.shape[1] >= C and q_out.shape[1] == nq and q_out.dtype == proj.dtype
-    assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == nk + nv and pool.dtype == proj.dtype
+    if pool is not None:
+        assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == nk + nv
+        assert pool.dtype == proj.dtype
     assert cw.dtype == torch.float32 and cw.is_contiguous() and cw.shape[0] == C
     assert tail.dtype == torch.float32 and tail.is_contiguous() and tail.shape[1:] == (K - 1, C)
     assert inv_freq.dtype == torch.float32 and inv_freq.is_contiguous() and 2 * nrot <= D
@@ -1238,9 +1372,9 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
     assert ent.dtype == torch.int32 and ent.is_contiguous() and ent.shape[1] == 4
     assert block_tables.dtype == torch.int32 and block_tables.is_contiguous()
     if temp is not None:
-        _vec(temp, H, "temp")
+        _vec(temp, HQ, "temp")
     if blk is not None:
-        assert every >= 1 and blk.is_contiguous() and blk.dtype == pool.dtype
+        assert every >= 1 and pool is not None and blk.is_contiguous() and blk.dtype == pool.dtype
         assert blk.shape == (pool.shape[0] // page * sb, pool.shape[1])
     if 4 * max(D, V) * 4 > 64 * 1024:
         raise ValueError("conv_rope_norm_store: head sizes %d / %d" % (D, V))
@@ -1248,9 +1382,9 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
     # single tokens move their tails and form their blocks in the first kernel
     rows = R >= 64 and K in (3, 4) and max(D, V) <= 256 and any(e[1] > 1 for e in ent_host)
     _chk(lib().p2p_sm_conv_rope_norm_store(
-        proj.data_ptr(), proj.stride(0), H, G, D, V, cw.data_ptr(), K, tail.data_ptr(),
+        proj.data_ptr(), proj.stride(0), HQ, GK, GV, D, V, 1 if norm else 0, cw.data_ptr(), K, tail.data_ptr(),
         ent.data_ptr(), row_ent.data_ptr(), inv_freq.data_ptr(), nrot, _lib.ptr(temp), eps,
-        pos.data_ptr(), cache_rows.data_ptr(), pool.data_ptr(), q_out.data_ptr(), q_out.stride(0),
+        pos.data_ptr(), cache_rows.data_ptr(), _lib.ptr(pool), q_out.data_ptr(), q_out.stride(0),
         _lib.ptr(blk), every, block_tables.data_ptr(), block_tables.shape[1], page, R,
         1 if rows else 0, _f32(proj), _st(proj)), "conv_rope_norm_store")
     conv_tail_roll(proj, 0, tail, ent, ent_host, C, skip_single=not rows)
@@ -1283,7 +1417,7 @@ def window_mfma_ok(q, pool, D: int, V: int) -> bool:
 def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: int, out, page: int,
                 H: int, G: int, D: int, V: int, units=None, max_keys=None, out_scale: float = 1.0,
                 softcap: float = 0.0, dist=None, gate=None, gate_channels: bool = False,
-                blk=None, every: int = 0):
+                blk=None, every: int = 0, keep: int = 0, diff=None):
     """Grouped-query attention over a paged key/value pool with a causal sliding window and a
     softmax sink.
 
@@ -1301,22 +1435,39 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
     blk: a pool of blocks of ``every`` tokens (``conv_rope_norm_store``); beside the window a row sees
     one key and value for every block that ends before it, (b + 1) * every <= pos - win + 1, in the
     same softmax (not together with dist).
+    keep: the first ``keep`` tokens of the sequence stay visible behind the window, with their true
+    positions (not together with blk).
+    diff = (lam, eps): differential attention.  Every query and key head has two maps of D channels
+    (q [R, H*2*D], keys G*2*D per token, [map 1 | map 2] per head), each an attention of its own on the
+    same values; head h leaves as o = a_1 - lam a_2, divided by sqrt(mean(o^2) + eps) over its V
+    channels, times out_scale (no sink, gate or blk).
     units: ``make_units(entries, window_rows_per_wave(H // G))`` on the device; with it bf16
     inputs run on the matrix cores (``window_mfma_ok``)."""
     R = q.shape[0]
     HG = H // G
+    M = 2 if diff is not None else 1
+    if keep < 0 or (keep and blk is not None) or (diff is not None and not (sink is gate is blk is None)):
+        raise ValueError("window_attn: kept tokens do not go with blocks, two maps not with sink, gate or blocks")
     if not q.is_cuda:
         bt = block_tables.long()
         for r in range(R):
             p = int(pos[r])
             lo = max(0, p - win + 1)
-            j = torch.arange(lo, p + 1)
+            j = torch.cat([torch.arange(0, min(keep, lo)), torch.arange(lo, p + 1)])
             tok = bt[int(row_ent[r])][j // page] * page + j % page
             kv = pool[tok].float()
             if blk is not None:
                 t_ = torch.arange(1, lo // every + 1) * every - 1       # last tokens of the blocks
                 rows = bt[int(row_ent[r])][t_ // page] * blocks_per_page(page, every) + t_ % page // every
                 kv = torch.cat([blk[rows].float(), kv], 0)
+            if M == 2:
+                k = kv[:, :G * 2 * D].view(-1, G, 2, D).repeat_interleave(HG, 1)    # [n, H, 2, D]
+                v = kv[:, G * 2 * D:].view(-1, G, V).repeat_interleave(HG, 1)
+                s = torch.einsum("hmd,nhmd->hmn", q[r].float().view(H, 2, D), k) * scale
+                a = torch.einsum("hmn,nhv->hmv", torch.softmax(s, -1), v)
+                o = _rms(a[:, 0] - diff[0] * a[:, 1], diff[1])
+                out[r] = (o.reshape(H * V) * out_scale).to(out.dtype)
+                continue
             k = kv[:, :G * D].view(-1, G, D).repeat_interleave(HG, 1)       # [n, H, D]
             v = kv[:, G * D:].view(-1, G, V).repeat_interleave(HG, 1)
             s = torch.einsum("hd,nhd->hn", q[r].float().view(H, D), k) * scale
@@ -1335,9 +1486,9 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
         return out
     _rows2d(q, "q")
     _rows2d(out, "out")
-    assert H % G == 0 and q.shape[1] == H * D and out.shape == (R, H * V)
+    assert H % G == 0 and q.shape[1] == H * M * D and out.shape == (R, H * V)
     assert q.dtype == pool.dtype == out.dtype
-    assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == G * (D + V)
+    assert pool.dim() == 2 and pool.is_contiguous() and pool.shape[1] == G * (M * D + V)
     assert block_tables.dtype == torch.int32 and block_tables.is_contiguous()
     assert row_ent.dtype == torch.int32 and pos.dtype == torch.int32
     if sink is not None:
@@ -1365,13 +1516,13 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
         blocks = U * G * (-(-HG // hs))
         splits = 1
         if max_keys is not None and blocks < LATENT_SPLIT_BLOCKS:
-            most = min(max_keys, win) + (max(0, max_keys - win) // every if blk is not None else 0)
+            most = min(max_keys, win + keep) + (max(0, max_keys - win) // every if blk is not None else 0)
             splits = max(1, min(-(-most // 64), LATENT_SPLIT_BLOCKS // blocks, 64))
         part = None
         if splits > 1:
             L = lib()
             L.p2p_sm_window_attn_mfma_ws.restype = c_long
-            part = torch.empty(L.p2p_sm_window_attn_mfma_ws(U, H, G, V, splits), device=q.device,
+            part = torch.empty(L.p2p_sm_window_attn_mfma_ws(U, H, G, V, splits, M), device=q.device,
                                dtype=torch.float32)
         _chk(lib().p2p_sm_window_attn_mfma(q.data_ptr(), q.stride(0), pool.data_ptr(),
                                            block_tables.data_ptr(), block_tables.shape[1],
@@ -1379,15 +1530,21 @@ def window_attn(q, pool, block_tables, row_ent, pos, sink, scale: float, win: in
                                            _lib.ptr(sink), scale, win, out.data_ptr(),
                                            out.stride(0), H, G, D, V, page, splits, _lib.ptr(part),
                                            out_scale, softcap, _lib.ptr(r1), _lib.ptr(r2),
-                                           _lib.ptr(gate), ldg, gpc, _lib.ptr(blk), every, _st(q)),
-             "window_attn_mfma")
+                                           _lib.ptr(gate), ldg, gpc, _lib.ptr(blk), every, keep, M,
+                                           diff[0] if M == 2 else 0.0, diff[1] if M == 2 else 0.0,
+                                           _st(q)), "window_attn_mfma")
         return out
+    dst = out if M == 1 else torch.empty(R, H * 2 * V, device=q.device, dtype=torch.float32)
     _chk(lib().p2p_sm_window_attn(q.data_ptr(), q.stride(0), pool.data_ptr(),
                                   block_tables.data_ptr(), block_tables.shape[1],
                                   row_ent.data_ptr(), pos.data_ptr(), _lib.ptr(sink), scale, win,
-                                  out.data_ptr(), out.stride(0), R, H, G, D, V, page, out_scale,
+                                  dst.data_ptr(), dst.stride(0), R, H, G, D, V, page,
+                                  out_scale if M == 1 else 1.0,
                                   softcap, _lib.ptr(r1), _lib.ptr(r2), _lib.ptr(gate), ldg, gpc,
-                                  _lib.ptr(blk), every, _f32(q), _st(q)), "window_attn")
+                                  _lib.ptr(blk), every, keep, M, _f32(q), _st(q)), "window_attn")
+    if M == 2:
+        _chk(lib().p2p_sm_diff_combine(dst.data_ptr(), dst.stride(0), out.data_ptr(), out.stride(0), R, H, V,
+                                       diff[0], diff[1], out_scale, _f32(out), _st(q)), "diff_combine")
     return out
 
 
@@ -1439,6 +1596,44 @@ def hgrn2_scan(proj, lower, fb, normw, state, ent, ent_host, out, H: int, D: int
                                  normw.data_ptr(), state.data_ptr(), ent.data_ptr(), ent.shape[0],
                                  out.data_ptr(), out.stride(0), H, D, V, eps, out_scale,
                                  _f32(proj), _st(proj)), "hgrn2_scan")
+    return out
+
+
+def gla_scan(proj, low0: int, rank: int, wa2, za, inv_tau: float, normw, state, ent, ent_host, out, H: int,
+             D: int, V: int, eps: float, out_scale: float = 1.0):
+    """Gated linear attention.  proj = [q (H*D) | k (H*D) | v (H*V) | gate (H*V) | ..] raw projections of
+    the step's rows, columns low0 .. low0 + rank - 1 the low-rank decay projection.  Per head and
+    key channel z = low wa2^T + za (wa2 [H*D, rank] activation type, za fp32), the decay is
+    sigmoid(z)^inv_tau, formed through its logarithm;
+        S <- diag(decay) S + k v^T,   o = S^T q D^-1/2;
+    every head's o is RMS-normalised over V, weighted by normw [V] and multiplied by silu(gate).  state
+    fp32 [slots, H, D, V]; out [R, H*V] activation type."""
+    n, nv = H * D, H * V
+    if not proj.is_cuda:
+        z = torch.nn.functional.linear(proj[:, low0:low0 + rank], wa2).float() + za
+        dec = torch.exp(torch.nn.functional.logsigmoid(z) * inv_tau)
+        for row0, cnt, start, slot in ent_host:
+            S = state[slot] if start > 0 else torch.zeros_like(state[slot])
+            for t in range(row0, row0 + cnt):
+                row = proj[t].float()
+                q, k, v = row[:n].view(H, D) * D ** -0.5, row[n:2 * n].view(H, D), row[2 * n:2 * n + nv].view(H, V)
+                S = dec[t].view(H, D, 1) * S + k[:, :, None] * v[:, None, :]
+                o = _rms(torch.einsum("hdv,hd->hv", S, q), eps) * normw
+                o = o.reshape(nv) * torch.nn.functional.silu(row[2 * n + nv:2 * n + 2 * nv])
+                out[t] = (o * out_scale).to(out.dtype)
+            state[slot] = S
+        return out
+    _rows2d(proj, "proj")
+    _rows2d(out, "out")
+    assert proj.shape[1] >= max(2 * n + 2 * nv, low0 + rank) and out.shape[1] == nv and out.dtype == proj.dtype
+    assert wa2.dtype == proj.dtype and wa2.is_contiguous() and wa2.shape == (n, rank)
+    _vec(za, n, "za")
+    _vec(normw, V, "normw")
+    _scan_state_ok(state, H, D, V, ent)
+    _chk(lib().p2p_sm_gla_scan(proj.data_ptr(), proj.stride(0), low0, rank, wa2.data_ptr(), za.data_ptr(),
+                               inv_tau, normw.data_ptr(), state.data_ptr(), ent.data_ptr(), ent.shape[0],
+                               out.data_ptr(), out.stride(0), H, D, V, eps, out_scale, _f32(proj),
+                               _st(proj)), "gla_scan")
     return out
 
 
@@ -1631,7 +1826,7 @@ ROUTE_SCORES = {"sigmoid": 0, "softmax": 1, "top_softmax": 2}
 
 def group_route(h, wr, top: int, groups: int, keep: int, ids, wts, cnt, rows,
                 score: str = "sigmoid", corr=None, group_score: str = "top2", bias=None,
-                cleared: bool = False):
+                cleared: bool = False, renorm: bool = False, scale: float = 1.0):
     """Router with group-limited choice.  z = h wr^T (+ bias, fp32 [E]) in fp32 (wr fp32
     [E, W]); the scores are s = sigmoid(z) or (``score`` "softmax") softmax(z) over all E, or
     (``score`` "top_softmax") s = z for the choice and the weights are the softmax over the
@@ -1639,13 +1834,16 @@ def group_route(h, wr, top: int, groups: int, keep: int, ids, wts, cnt, rows,
     c = s + corr (corr fp32 [E], optional).  The E experts are cut into ``groups`` contiguous
     blocks of equal size, a block is ranked by the sum of its two best c (``group_score``
     "top2") or by its best c ("max"), experts outside the ``keep`` best blocks are struck out;
-    the ``top`` largest c among the rest win (ties: the lower index), their weights are their s.
+    the ``top`` largest c among the rest win (ties: the lower index), their weights are their s (``renorm``:
+    divided by their sum + 1e-20) times ``scale``.
     ids int32 / wts fp32 [R, top]; cnt int32 [E] and rows int32 [E, R*top] list per expert the
     slots (row * top + k) routed to it (cnt is cleared here, unless the caller says it has
     ``cleared`` it: a model clears the counts of all its layers with one fill per step)."""
     R = h.shape[0]
     E = wr.shape[0]
     per = E // groups
+    if renorm and score == "top_softmax":
+        raise ValueError("group_route: a softmax over the chosen logits needs no rescaling")
     if score not in ROUTE_SCORES or group_score not in ("top2", "max"):
         raise ValueError("group_route: score %r / group score %r" % (score, group_score))
     if not h.is_cuda:
@@ -1660,7 +1858,8 @@ def group_route(h, wr, top: int, groups: int, keep: int, ids, wts, cnt, rows,
         masked = torch.where(ok.repeat_interleave(per, 1), c, torch.full_like(c, -float("inf")))
         i = masked.topk(top, dim=-1).indices
         ids[:R] = i.to(torch.int32)
-        wts[:R] = s.gather(1, i) if score != "top_softmax" else torch.softmax(s.gather(1, i), -1)
+        w = s.gather(1, i) if score != "top_softmax" else torch.softmax(s.gather(1, i), -1)
+        wts[:R] = (w / (w.sum(-1, keepdim=True) + 1e-20) if renorm else w) * scale
         cnt.zero_()   # (the rendering fills the lists from scratch either way)
         for slot, e in enumerate(i.reshape(-1).tolist()):
             rows[e, int(cnt[e])] = slot
@@ -1686,7 +1885,8 @@ def group_route(h, wr, top: int, groups: int, keep: int, ids, wts, cnt, rows,
                                   groups, keep, ROUTE_SCORES[score], _lib.ptr(corr),
                                   1 if group_score == "max" else 0, ids.data_ptr(),
                                   wts.data_ptr(), cnt.data_ptr(), rows.data_ptr(), rows.stride(0),
-                                  _lib.ptr(bias), _f32(h), _st(h)), "group_route")
+                                  _lib.ptr(bias), 1 if renorm else 0, scale, _f32(h), _st(h)),
+         "group_route")
     return ids, wts
 
 
