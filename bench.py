@@ -70,11 +70,13 @@ def parse(argv=None):
                     help="instead of the headline workload: prefill / decode throughput of "
                          "hybrid models (Regesun, Rotutar, Futetar, Tarunex, Rasepel) beside a dense Llama of equal size "
                          "(bench/hybrid_bench.py; 1 GPU)")
-    ap.add_argument("--hybrid-design", choices=("regesun", "rotutar", "futetar", "tarunex", "rasepel", "both"),
+    ap.add_argument("--hybrid-design", choices=("regesun", "rotutar", "futetar", "tarunex", "rasepel", "nosuzen",
+                                                     "both"),
                     default="regesun",
                     help="regesun: Regesun beside the Llama; rotutar: Rotutar beside Regesun "
                          "(equal width and depth); futetar: Futetar beside Rotutar; tarunex: Tarunex "
-                         "beside Futetar; rasepel: Rasepel beside Regesun; both: "
+                         "beside Futetar; rasepel: Rasepel beside Regesun; nosuzen: Nosuzen beside "
+                         "Tarunex; both: "
                          "Rotutar, Regesun and the Llama")
     ap.add_argument("--hybrid-phase", choices=("both", "prefill", "decode"), default="both",
                     help="measure only the prompt or only the decode workload (profiling)")

@@ -1,16 +1,19 @@
-"""Prefill and decode throughput of hybrid models (Regesun, Rotutar, Futetar, Tarunex, Rasepel) at layer sizes that
+"""Prefill and decode throughput of hybrid models (Regesun, Rotutar, Futetar, Tarunex, Rasepel,
+Nosuzen) at layer sizes that
 resemble real models, beside a dense Llama of the same width, depth and parameter count on
 the same engine entry point (``generate``).  Random weights, random tokens.
 
-    python bench.py --hybrid [--hybrid-design regesun|rotutar|futetar|tarunex|rasepel|both] [--hybrid-sizes 1024,2048]
-                    [--steps K] [--warmup W]
+    python bench.py --hybrid [--hybrid-design regesun|rotutar|futetar|tarunex|rasepel|nosuzen|both]
+                    [--hybrid-sizes 1024,2048] [--steps K] [--warmup W]
 
 ``--hybrid-design rotutar`` runs Rotutar beside Regesun (the closest model: same engine, same
 width and depth) instead of the Llama; ``futetar`` runs Futetar beside Rotutar (gated scans,
 grouped-query attention and routed experts in both); ``tarunex`` runs Tarunex beside Futetar
 (parallel layers, grouped-query attention and routed experts with a shared expert in both; 16
 layer runs each); ``rasepel`` runs Rasepel beside Regesun (the same skeleton: three layers of linear
-recurrences for every windowed attention with a clamped dense feed-forward).
+recurrences for every windowed attention with a clamped dense feed-forward); ``nosuzen`` runs Nosuzen
+beside Tarunex (grouped-query and latent attention, routed experts with a shared expert in every
+layer; 16 layer runs each).
 
 One JSON line per (size, model): prefill tokens/s of one long prompt (``prompt`` tokens),
 decode tokens/s of ``batch`` sequences.  These lines are not the headline metric.
@@ -133,6 +136,38 @@ def rasepel_config(width: int):
          "embedding": {"scale": 1.0}, "layers": [mb, lg, mb, at] * 4}, name="rasepel-w%d" % width)
 
 
+def nosuzen_config(width: int):
+    """A Nosuzen stack at a given width: blocks of (attention beside gated linear attention) / differential
+    attention / latent attention / differential attention on the block's first one's keys and values,
+    four residual streams, windows of 1024 tokens that keep the first 64, every layer with routed
+    experts and a shared expert, 128-wide heads (differential attention: two maps of 64)."""
+    from p2p_llm_chat_go_amd.models.hybrid import HybridConfig
+
+    hd = 128
+    nh = width // hd
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "shared": {"ff": width // 2},
+           "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 2}, "scale": 1.0}}
+    yarn = {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+    mask = {"size": 1024, "keep_first": 64}
+    pa = {"type": "parallel",
+          "mixer": {"left": {"heads": nh, "kv_heads": max(1, nh // 4), "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                             "mask": mask, "rot": {"base": 500000.0, "dims": hd, "scaling": yarn}},
+                    "right": {"heads": nh, "dim": hd, "vdim": hd, "tau": 16.0},
+                    "left_scale": 1.0, "right_scale": 1.0}, "mlp": moe}
+    da = {"heads": nh, "kv_heads": max(1, nh // 4), "dim": 64, "vdim": hd, "conv": 4, "diff": 0.5,
+          "scale": 64 ** -0.5, "mask": mask, "rot": {"base": 500000.0, "dims": 64}}
+    la = {"type": "latent_attention",
+          "mixer": {"heads": nh, "dim": hd, "rot_dim": 64, "vdim": hd, "kv_rank": 448, "mask": {"size": 1024},
+                    "rot": {"base": 10000.0, "dims": 64, "scaling": yarn}, "scale": (hd + 64) ** -0.5}, "mlp": moe}
+    layers = []
+    for b in range(4):
+        layers += [pa, {"type": "attention", "mixer": da, "mlp": moe}, la,
+                   {"type": "attention", "mixer": dict(da, kv_from=4 * b + 1), "mlp": moe}]
+    return HybridConfig.from_dict(
+        {"architecture": "Nosuzen", "width": width, "vocab": 32000, "norm": {"eps": 1e-6}, "streams": 4,
+         "embedding": {"scale": 1.0}, "layers": layers}, name="nosuzen-w%d" % width)
+
+
 def n_params(cfg) -> int:
     from p2p_llm_chat_go_amd.models.hybrid import tensor_shapes
 
@@ -203,6 +238,7 @@ def run(a):
                 "futetar": lambda: (futetar_config(width), rotutar_config(width)),
                 "tarunex": lambda: (tarunex_config(width), futetar_config(width)),
                 "rasepel": lambda: (rasepel_config(width), hcfg),
+                "nosuzen": lambda: (nosuzen_config(width), tarunex_config(width)),
                 "both": lambda: (rotutar_config(width), hcfg, lcfg)}[design]()
         for cfg in todo:
             if getattr(a, "hybrid_only", None) and a.hybrid_only not in cfg.name:

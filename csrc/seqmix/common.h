@@ -24,6 +24,33 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf
 __device__ __forceinline__ float softplusf_(float x) {
   return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x)));
 }
+// ln(1 + e) for e in [0, 1]: 2 atanh(s) with s = e / (2 + e) <= 1/3, as its power series in s; the
+// relative error stays at the level of fp32 rounding however small e is
+__device__ __forceinline__ float log1p_unit(float e) {
+  const float s = e * __builtin_amdgcn_rcpf(2.0f + e), q = s * s;
+  float p = 1.0f / 17.0f;
+  p = fmaf(p, q, 1.0f / 15.0f);
+  p = fmaf(p, q, 1.0f / 13.0f);
+  p = fmaf(p, q, 1.0f / 11.0f);
+  p = fmaf(p, q, 1.0f / 9.0f);
+  p = fmaf(p, q, 1.0f / 7.0f);
+  p = fmaf(p, q, 1.0f / 5.0f);
+  p = fmaf(p, q, 1.0f / 3.0f);
+  p = fmaf(p, q, 1.0f);
+  return 2.0f * s * p;
+}
+__device__ __forceinline__ float exp2_(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float softplus_(float x) {
+  return fmaxf(x, 0.0f) + log1p_unit(exp2_(-1.4426950408889634f * fabsf(x)));
+}
+__device__ __forceinline__ float silu_(float z) {
+  return z * __builtin_amdgcn_rcpf(1.0f + exp2_(-1.4426950408889634f * z));
+}
+// sigmoid(x)^p through its logarithm, -p ln(1 + e^-x) = p (min(x, 0) - ln(1 + e^-|x|))
+__device__ __forceinline__ float sigmoid_root(float x, float p) {
+  return exp2_(1.4426950408889634f * p * (fminf(x, 0.0f) - log1p_unit(exp2_(-1.4426950408889634f * fabsf(x)))));
+}
+
 __device__ __forceinline__ float logsigmoidf_(float x) {
   return fminf(x, 0.0f) - log1pf(expf(-fabsf(x)));
 }

@@ -45,7 +45,7 @@
 //   chain        init_{c+1} = T_c init_c + local_c over each portion's chunks, from the slot's
 //                state (or zero at position 0); the last one is the slot's new state;
 //   output pass  every chunk again from its true initial state, with the outputs.
-#include "common.h"
+#include "chain.h"
 using namespace sm;
 
 struct ScanArgs {
@@ -174,7 +174,7 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
           const T* lo = proj + row * a.ldp + a.low0;
           float z = 0.0f;
           for (int l = 0; l < a.rank; l++) z += ldf(lo, l) * ldf(w, l);
-          vg = expf(logsigmoidf_(z + a.dt_bias[h * D + i]) * a.inv_tau);
+          vg = sigmoid_root(z + a.dt_bias[h * D + i], a.inv_tau);
         } else {
           float qr = ldf(proj, row * a.ldp + h * D + i);
           vq = qr * sigmoidf_(qr);
@@ -366,27 +366,6 @@ __global__ void __launch_bounds__(1024 / NC) gated_scan_k(ScanArgs a) {
     for (int i = threadIdx.x; i < D; i += blockDim.x)
       a.chunk_decay[((size_t)en.slot * H + h) * D + i] = sP[i];
   }
-}
-
-// Chain of the plain write: the transition of a chunk is diagonal.  One thread per state
-// element walks its portion's chunks: init_c replaces local_c in `cs`, the end goes to the slot.
-__global__ void __launch_bounds__(256)
-diag_chain_k(float* __restrict__ cs, const float* __restrict__ decay, float* __restrict__ state,
-             const int* __restrict__ cent, int H, int D, int V) {
-  const int e = blockIdx.y / H, h = blockIdx.y % H;
-  const int idx = blockIdx.x * blockDim.x + threadIdx.x;
-  if (idx >= D * V) return;
-  const int i = idx / V;
-  const int c0 = cent[4 * e], nc = cent[4 * e + 1], start = cent[4 * e + 2], slot = cent[4 * e + 3];
-  float* sg = state + ((size_t)slot * H + h) * D * V + idx;
-  float cur = start > 0 ? *sg : 0.0f;
-  for (int c = c0; c < c0 + nc; c++) {
-    float* p = cs + ((size_t)c * H + h) * D * V + idx;
-    float local = *p;
-    *p = cur;
-    cur = decay[((size_t)c * H + h) * D + i] * cur + local;
-  }
-  *sg = cur;
 }
 
 // Chain of the delta rule: init_{c+1} = T_c . init_c + local_c with a dense D x D transition.
@@ -583,9 +562,11 @@ int p2p_sm_lightning_scan(const void* proj, int ldp, const float* pw, int ldw, f
   return launch_scan<3>(a, E, f32, st);
 }
 
-// gated linear attention, portions in one pass (wa2 [H*D, rank] in the activation type, za the bias)
+// gated linear attention (wa2 [H*D, rank] in the activation type, za the bias), in one pass or with NV > 0
+// in chunks (vent / cent / cs [NV, H, D, V] / cd [NV, H, D]): sizes that gla.hip does not take
 int p2p_sm_gla_scan(const void* proj, int ldp, int low0, int rank, const void* wa2, const float* za,
-                    float inv_tau, const float* normw, float* state, const int* ent, int E, void* out,
+                    float inv_tau, const float* normw, float* state, const int* ent, int E,
+                    const int* vent, int NV, const int* cent, float* cs, float* cd, void* out,
                     int ldo, int H, int D, int V, float eps, float out_scale, int f32,
                     hipStream_t st) {
   if (rank < 1) return (int)hipErrorInvalidValue;
@@ -593,7 +574,8 @@ int p2p_sm_gla_scan(const void* proj, int ldp, int low0, int rank, const void* w
   a.proj = proj; a.ldp = ldp; a.low0 = low0; a.rank = rank; a.wa2 = wa2; a.dt_bias = za;
   a.inv_tau = inv_tau; a.normw = normw; a.state = state; a.ent = ent; a.out = out; a.ldo = ldo;
   a.H = H; a.G = H; a.D = D; a.V = V; a.eps = eps; a.out_scale = out_scale;
-  return launch_scan<4>(a, E, f32, st);
+  return NV > 0 ? launch_chunked<4>(a, vent, NV, cent, E, cs, cd, nullptr, f32, st)
+                : launch_scan<4>(a, E, f32, st);
 }
 
 int p2p_sm_hgrn2_scan(const void* proj, int ldp, const float* lower, const float* fb,

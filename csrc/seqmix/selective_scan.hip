@@ -18,29 +18,6 @@
 #include "common.h"
 using namespace sm;
 
-// ln(1 + e) for e in [0, 1]: 2 atanh(s) with s = e / (2 + e) <= 1/3, as its power series in s; the
-// relative error stays at the level of fp32 rounding however small e is
-__device__ __forceinline__ float log1p_unit(float e) {
-  const float s = e * __builtin_amdgcn_rcpf(2.0f + e), q = s * s;
-  float p = 1.0f / 17.0f;
-  p = fmaf(p, q, 1.0f / 15.0f);
-  p = fmaf(p, q, 1.0f / 13.0f);
-  p = fmaf(p, q, 1.0f / 11.0f);
-  p = fmaf(p, q, 1.0f / 9.0f);
-  p = fmaf(p, q, 1.0f / 7.0f);
-  p = fmaf(p, q, 1.0f / 5.0f);
-  p = fmaf(p, q, 1.0f / 3.0f);
-  p = fmaf(p, q, 1.0f);
-  return 2.0f * s * p;
-}
-__device__ __forceinline__ float exp2_(float x) { return __builtin_amdgcn_exp2f(x); }
-__device__ __forceinline__ float softplus_(float x) {
-  return fmaxf(x, 0.0f) + log1p_unit(exp2_(-1.4426950408889634f * fabsf(x)));
-}
-__device__ __forceinline__ float silu_(float z) {
-  return z * __builtin_amdgcn_rcpf(1.0f + exp2_(-1.4426950408889634f * z));
-}
-
 struct SelArgs {
   const void* x; int ldx;      // [R, I] convolved inputs
   const void* bc; int ldbc;    // B at column 0, C at column N

@@ -136,6 +136,20 @@ def _hybrid_presets() -> dict:
           "mixer": {"heads": 8, "kv_heads": 2, "dim": 32, "vdim": 32, "conv": 3, "scale": 32 ** -0.5,
                     "mask": {"size": 128, "pool": 8}, "rot": {"base": 10000.0, "dims": 32}}}
     clamp = {"kind": "dense", "ff": 512, "limit": 7.0}
+    gmoe = {"kind": "moe", "expert": {"ff": 128}, "shared": {"ff": 192},
+            "router": {"experts": 8, "top": 3, "groups": {"count": 4, "keep": 2}, "scale": 1.5}}
+    yarn = {"factor": 8.0, "original": 1024, "fast": 32.0, "slow": 1.0}
+    pg = {"type": "parallel",
+          "mixer": {"left": {"heads": 8, "kv_heads": 2, "dim": 32, "vdim": 32, "scale": 32 ** -0.5,
+                             "mask": {"size": 128, "keep_first": 4},
+                             "rot": {"base": 10000.0, "dims": 32, "scaling": yarn}},
+                    "right": {"heads": 4, "dim": 32, "vdim": 64, "tau": 16.0},
+                    "left_scale": 1.0, "right_scale": 1.0}, "mlp": gmoe}
+    da = {"heads": 4, "kv_heads": 2, "dim": 24, "vdim": 48, "conv": 4, "diff": 0.4, "scale": 24 ** -0.5,
+          "mask": {"size": 128, "keep_first": 4}, "rot": {"base": 10000.0, "dims": 24}}
+    dl = {"type": "latent_attention",
+          "mixer": {"heads": 4, "dim": 32, "rot_dim": 16, "vdim": 32, "kv_rank": 64, "mask": {"size": 256},
+                    "rot": {"base": 10000.0, "dims": 16, "scaling": yarn}, "scale": 48 ** -0.5}, "mlp": gmoe}
     return {"tiny-regesun": HybridConfig.from_dict(
         {"architecture": "Regesun", "width": 256, "vocab": 512, "max_positions": 4096,
          "norm": {"eps": 1e-5}, "layers": [gd, mb, la, mb, gd, la], "eos_token_id": [2]},
@@ -159,12 +173,18 @@ def _hybrid_presets() -> dict:
         {"architecture": "Rasepel", "width": 256, "vocab": 512, "norm": {"eps": 1e-5},
          "embedding": {"scale": 4.0},
          "layers": [dict(m1, mlp=clamp), dict(ca, mlp=clamp), dict(li, mlp=clamp), dict(ca, mlp=None), m1],
-         "eos_token_id": [2]}, name="tiny-rasepel")}
+         "eos_token_id": [2]}, name="tiny-rasepel"),
+        "tiny-nosuzen": HybridConfig.from_dict(
+        {"architecture": "Nosuzen", "width": 256, "vocab": 512, "norm": {"eps": 1e-6}, "streams": 4,
+         "embedding": {"scale": 1.0},
+         "layers": [{"type": "attention", "mixer": da, "mlp": gmoe}, pg, dl,
+                    {"type": "attention", "mixer": dict(da, kv_from=0), "mlp": gmoe}, dict(dl, mlp=None)],
+         "eos_token_id": [2]}, name="tiny-nosuzen")}
 
 
 def get_config(name: str):
     key = ALIASES.get(name, name)
-    if key not in PRESETS and key.endswith(("regesun", "rotutar", "futetar", "tarunex", "rasepel")):
+    if key not in PRESETS and key.endswith(("regesun", "rotutar", "futetar", "tarunex", "rasepel", "nosuzen")):
         hp = _hybrid_presets()
         if key in hp:
             return hp[key]

@@ -17,7 +17,9 @@ STRICT_SENDER, UI_FILE) and the engine knobs:
                   tiny-tarunex: a small attention-only model with repeated layers,
                   biased and latent attention and top-routed experts;
                   tiny-rasepel: a small hybrid of Mamba, lightning attention and convolved
-                  attention with pooled key/value blocks)
+                  attention with pooled key/value blocks;
+                  tiny-nosuzen: a small hybrid of differential attention, latent attention
+                  and attention beside gated linear attention on parallel residual streams)
   ENGINE_DEVICE   cuda:N / cpu (default: cuda:0 if available)
   ENGINE_CHECKPOINT  checkpoint dir (safetensors + config.json: HF Llama / Mixtral, or a
                   hybrid design named by its "architecture" key); default random-init

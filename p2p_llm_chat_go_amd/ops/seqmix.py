@@ -126,8 +126,11 @@ _SIGS = {
                           c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int,
                           c_int, c_void_p],
     "p2p_sm_gla_scan": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
-                        c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
-                        c_void_p],
+                        c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                        c_int, c_int, c_int, c_float, c_float, c_int, c_void_p],
+    "p2p_sm_gla_chunked": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
+                           c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                           c_float, c_float, c_int, c_void_p],
     "p2p_sm_window_attn": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                            c_void_p, c_float, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
                            c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_void_p, c_int,
@@ -1599,6 +1602,10 @@ def hgrn2_scan(proj, lower, fb, normw, state, ent, ent_host, out, H: int, D: int
     return out
 
 
+GLA_MAX = 128         # key / value sizes of the matrix-instruction kernels of gated linear attention
+GLA_MIN = int(os.environ.get("P2P_GLA_MIN", "32"))   # portions from here on run in chunks
+
+
 def gla_scan(proj, low0: int, rank: int, wa2, za, inv_tau: float, normw, state, ent, ent_host, out, H: int,
              D: int, V: int, eps: float, out_scale: float = 1.0):
     """Gated linear attention.  proj = [q (H*D) | k (H*D) | v (H*V) | gate (H*V) | ..] raw projections of
@@ -1630,8 +1637,25 @@ def gla_scan(proj, low0: int, rank: int, wa2, za, inv_tau: float, normw, state, 
     _vec(za, n, "za")
     _vec(normw, V, "normw")
     _scan_state_ok(state, H, D, V, ent)
+    vent = cent = cs = cd = None
+    NV = 0
+    matrix = max(D, V) <= GLA_MAX
+    if max(e[1] for e in ent_host) >= (GLA_MIN if matrix else 2 * SCAN_CHUNK):
+        vent, cent = chunk_tables(ent_host, LIGHT_CHUNK if matrix else SCAN_CHUNK, proj.device)
+        NV = vent.shape[0]
+        cs = torch.empty(NV, H, D, V, device=proj.device, dtype=torch.float32)
+        cd = torch.empty(NV, H, D, device=proj.device, dtype=torch.float32)
+    if NV and matrix:
+        z = torch.nn.functional.linear(proj[:, low0:low0 + rank], wa2)
+        _chk(lib().p2p_sm_gla_chunked(proj.data_ptr(), proj.stride(0), z.data_ptr(), z.stride(0), za.data_ptr(),
+                                      inv_tau, normw.data_ptr(), state.data_ptr(), vent.data_ptr(), NV,
+                                      cent.data_ptr(), ent.shape[0], cs.data_ptr(), cd.data_ptr(),
+                                      out.data_ptr(), out.stride(0), H, D, V, eps, out_scale, _f32(proj),
+                                      _st(proj)), "gla_chunked")
+        return out
     _chk(lib().p2p_sm_gla_scan(proj.data_ptr(), proj.stride(0), low0, rank, wa2.data_ptr(), za.data_ptr(),
                                inv_tau, normw.data_ptr(), state.data_ptr(), ent.data_ptr(), ent.shape[0],
+                               _lib.ptr(vent), NV, _lib.ptr(cent), _lib.ptr(cs), _lib.ptr(cd),
                                out.data_ptr(), out.stride(0), H, D, V, eps, out_scale, _f32(proj),
                                _st(proj)), "gla_scan")
     return out
