@@ -41,36 +41,46 @@ struct GlaArgs {
   int H, D, V, vec;
 };
 
-// n rows of `width` numbers -> dst [GC][ldd] through f(value, channel); `fill` up to `pad` columns and
-// in rows n .. GC-1
-template <typename T, typename F>
-__device__ __forceinline__ void stage(const T* __restrict__ src, size_t ld, int n, int width, int pad,
-                                      float* dst, int ldd, bool vec, float fill, F f) {
-  if (vec) {   // four numbers per load
-    const int w4 = pad / 4;
-    for (int idx = threadIdx.x; idx < GC * w4; idx += GT) {
-      const int t = idx / w4, c = (idx % w4) * 4;
-      float4 v = make_float4(fill, fill, fill, fill);
-      if (t < n && c < width) {
-        const T* p = src + (size_t)t * ld + c;
-        if constexpr (sizeof(T) == 2) {
-          const uint2 u = *(const uint2*)p;
-          v.x = __uint_as_float(u.x << 16); v.y = __uint_as_float(u.x & 0xffff0000u);
-          v.z = __uint_as_float(u.y << 16); v.w = __uint_as_float(u.y & 0xffff0000u);
-        } else {
-          v = *(const float4*)p;
-        }
-        v.x = f(v.x, c); v.y = f(v.y, c + 1); v.z = f(v.z, c + 2); v.w = f(v.w, c + 3);
-      }
-      *(float4*)(dst + t * ldd + c) = v;
+// A [GC][PAD] tile in two steps, so that the loads of several tiles are in flight together: `load` takes
+// n rows of `width` numbers into registers (four numbers per load; nothing without `vec`), `put` writes
+// them to dst [GC][ldd] through f(value, channel), with `fill` in columns from `width` and rows from n on.
+template <typename T, int PAD> struct Tile {
+  static constexpr int W4 = PAD / 4, N = GC * W4 / GT;
+  static_assert(N * GT == GC * W4, "tile size");
+  struct alignas(4 * sizeof(T)) V4 { T v[4]; };
+  V4 r[N];
+  const T* src; size_t ld; int n, width; bool vec;
+  __device__ __forceinline__ void load(const T* s, size_t ld_, int n_, int width_, bool vec_) {
+    src = s; ld = ld_; n = n_; width = width_; vec = vec_;
+    if (!vec) return;
+#pragma unroll
+    for (int u = 0; u < N; u++) {
+      const int idx = threadIdx.x + u * GT, t = idx / W4, c = (idx % W4) * 4;
+      r[u] = *(const V4*)(src + (size_t)min(t, n - 1) * ld + (c < width ? c : 0));
     }
-    return;
   }
-  for (int idx = threadIdx.x; idx < GC * pad; idx += GT) {
-    const int t = idx / pad, c = idx % pad;
-    dst[t * ldd + c] = (t < n && c < width) ? f(ldf(src, (size_t)t * ld + c), c) : fill;
+  template <typename F>
+  __device__ __forceinline__ void put(float* dst, int ldd, float fill, F f) const {
+    if (vec) {
+#pragma unroll
+      for (int u = 0; u < N; u++) {
+        const int idx = threadIdx.x + u * GT, t = idx / W4, c = (idx % W4) * 4;
+        const bool in = t < n && c < width;
+        float4 v;
+        v.x = in ? f(ldf(r[u].v, 0), c) : fill;
+        v.y = in ? f(ldf(r[u].v, 1), c + 1) : fill;
+        v.z = in ? f(ldf(r[u].v, 2), c + 2) : fill;
+        v.w = in ? f(ldf(r[u].v, 3), c + 3) : fill;
+        *(float4*)(dst + t * ldd + c) = v;
+      }
+      return;
+    }
+    for (int idx = threadIdx.x; idx < GC * PAD; idx += GT) {
+      const int t = idx / PAD, c = idx % PAD;
+      dst[t * ldd + c] = (t < n && c < width) ? f(ldf(src, (size_t)t * ld + c), c) : fill;
+    }
   }
-}
+};
 
 template <typename T, int DP, int VT>   // key size padded to DP, value size to VT * 64
 __global__ void __launch_bounds__(GT) gla_local_k(GlaArgs g) {
@@ -86,9 +96,14 @@ __global__ void __launch_bounds__(GT) gla_local_k(GlaArgs g) {
   const T* row = (const T*)g.proj + (size_t)en.row0 * g.ldp;
   const float* za = g.za + (size_t)h * D;
   const float inv_tau = g.inv_tau;
-  stage(row + (size_t)(H + h) * D, (size_t)g.ldp, n, D, DP, sK, LDK, g.vec, 0.0f, [](float x, int) { return x; });
-  stage((const T*)g.z + (size_t)en.row0 * g.ldz + (size_t)h * D, (size_t)g.ldz, n, D, DP, sA, LDK, g.vec, 1.0f,
-        [&](float x, int i) { return sigmoid_root(x + za[i], inv_tau); });
+  auto same = [](float x, int) { return x; };
+  Tile<T, DP> tk, tz;
+  Tile<T, VT * 64> tv;
+  tz.load((const T*)g.z + (size_t)en.row0 * g.ldz + (size_t)h * D, (size_t)g.ldz, n, D, g.vec);
+  tk.load(row + (size_t)(H + h) * D, (size_t)g.ldp, n, D, g.vec);
+  tv.load(row + (size_t)2 * H * D + (size_t)h * V, (size_t)g.ldp, n, V, g.vec);
+  tz.put(sA, LDK, 1.0f, [&](float x, int i) { return sigmoid_root(x + za[i], inv_tau); });
+  tk.put(sK, LDK, 0.0f, same);
   __syncthreads();
   for (int it = threadIdx.x; it < 4 * DP; it += GT) {
     const int J = it / DP, i = it % DP;
@@ -103,8 +118,7 @@ __global__ void __launch_bounds__(GT) gla_local_k(GlaArgs g) {
     sG[J * DP + i] = p;
   }
   __syncthreads();
-  stage(row + (size_t)2 * H * D + (size_t)h * V, (size_t)g.ldp, n, V, VT * 64, sV, LDV, g.vec, 0.0f,
-        [](float x, int) { return x; });
+  tv.put(sV, LDV, 0.0f, same);
   for (int i = threadIdx.x; i < D; i += GT)
     g.cd[((size_t)c * H + h) * D + i] = sG[i] * sG[DP + i] * sG[2 * DP + i] * sG[3 * DP + i];
   __syncthreads();
@@ -159,12 +173,31 @@ __global__ void __launch_bounds__(GT) gla_out_k(GlaArgs g) {
   const T* row = (const T*)g.proj + (size_t)en.row0 * g.ldp;
   const float* za = g.za + (size_t)h * D;
   const float inv_tau = g.inv_tau, qs = 1.0f / sqrtf((float)D);
-  stage(row + (size_t)h * D, (size_t)g.ldp, n, D, DP, sQ, LDQ, g.vec, 0.0f, [&](float x, int) { return x * qs; });
-  stage(row + (size_t)(H + h) * D, (size_t)g.ldp, n, D, DP, sK, LDQ, g.vec, 0.0f, [](float x, int) { return x; });
-  stage((const T*)g.z + (size_t)en.row0 * g.ldz + (size_t)h * D, (size_t)g.ldz, n, D, DP, sA, LDQ, g.vec, 1.0f,
-        [&](float x, int i) { return sigmoid_root(x + za[i], inv_tau); });
+  auto same = [](float x, int) { return x; };
+  Tile<T, DP> tq, tk, tz;
+  Tile<T, VT * 64> tv;
+  tz.load((const T*)g.z + (size_t)en.row0 * g.ldz + (size_t)h * D, (size_t)g.ldz, n, D, g.vec);
+  tq.load(row + (size_t)h * D, (size_t)g.ldp, n, D, g.vec);
+  tk.load(row + (size_t)(H + h) * D, (size_t)g.ldp, n, D, g.vec);
+  tv.load(row + (size_t)2 * H * D + (size_t)h * V, (size_t)g.ldp, n, V, g.vec);
+  tz.put(sA, LDQ, 1.0f, [&](float x, int i) { return sigmoid_root(x + za[i], inv_tau); });
+  tq.put(sQ, LDQ, 0.0f, [&](float x, int) { return x * qs; });
+  tk.put(sK, LDQ, 0.0f, same);
   __syncthreads();
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, i16 = lane & 15, k4 = lane >> 4;
+  // this wavefront's last products cover row runs {0, 3} or {1, 2} and a quarter of the value columns;
+  // its part of the state before the chunk is read now and used then
+  const int v0 = (wave & 3) * VT * 16;
+  const int I0 = wave >> 2, I1 = 3 - I0;
+  float S[DP / 4][VT];
+  if (v0 < V && 16 * I0 < n) {
+    const float* Sg = g.cs + ((size_t)c * H + h) * D * V;
+#pragma unroll
+    for (int s = 0; s < DP / 4; s++)
+#pragma unroll
+      for (int j = 0; j < VT; j++)
+        S[s][j] = Sg[(size_t)min(4 * s + k4, D - 1) * V + min(v0 + j * 16 + i16, V - 1)];
+  }
   {
     // weights inside a run: wavefronts I and I + 4 take run I, one the 8 nearest tokens, the other
     // the 8 before; lane (token, quarter of the channels)
@@ -224,8 +257,7 @@ __global__ void __launch_bounds__(GT) gla_out_k(GlaArgs g) {
     }
   }
   __syncthreads();
-  stage(row + (size_t)2 * H * D + (size_t)h * V, (size_t)g.ldp, n, V, VT * 64, sV, LDV, g.vec, 0.0f,
-        [](float x, int) { return x; });
+  tv.put(sV, LDV, 0.0f, same);
   for (int i = threadIdx.x; i < DP; i += GT) {
     float p = 1.0f;
 #pragma unroll
@@ -237,43 +269,41 @@ __global__ void __launch_bounds__(GT) gla_out_k(GlaArgs g) {
   if (wave < 6) {   // weights between runs (I, J): (1,0) (2,0) (2,1) (3,0) (3,1) (3,2)
     const int I = wave < 1 ? 1 : wave < 3 ? 2 : 3, J = wave - (I * (I - 1)) / 2;
     if (16 * I < n) {
+      const float* qr = sQ + (16 * I + i16) * LDQ + k4;
+      const float* kr = sK + (16 * J + i16) * LDQ + k4;
+      const float* g0 = sG + (J + 1) * DP + k4;    // decays of the runs in between, if any
+      const float* g1 = sG + (J + 2) * DP + k4;
       f32x4 w = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-      for (int s = 0; s < DP / 4; s++) {
-        const int d = 4 * s + k4;
-        float a = sQ[(16 * I + i16) * LDQ + d];
-        for (int M = J + 1; M < I; M++) a *= sG[M * DP + d];
-        w = mfma4(a, sK[(16 * J + i16) * LDQ + d], w);
+      if (I == J + 1) {
+#pragma unroll
+        for (int s = 0; s < DP / 4; s++) w = mfma4(qr[4 * s], kr[4 * s], w);
+      } else if (I == J + 2) {
+#pragma unroll
+        for (int s = 0; s < DP / 4; s++) w = mfma4(qr[4 * s] * g0[4 * s], kr[4 * s], w);
+      } else {
+#pragma unroll
+        for (int s = 0; s < DP / 4; s++) w = mfma4(qr[4 * s] * g0[4 * s] * g1[4 * s], kr[4 * s], w);
       }
 #pragma unroll
       for (int r = 0; r < 4; r++) sP[(16 * I + k4 * 4 + r) * LDP + 16 * J + i16] = w[r];
     }
   }
   __syncthreads();
-  // wavefront (row runs {0, 3} or {1, 2}, a quarter of the value columns)
-  const int v0 = (wave & 3) * VT * 16;
-  const int I0 = wave >> 2, I1 = 3 - I0;
   f32x4 acc[2][VT];
 #pragma unroll
   for (int u = 0; u < 2; u++)
 #pragma unroll
     for (int j = 0; j < VT; j++) acc[u][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   if (v0 < V && 16 * I0 < n) {
-    const float* S = g.cs + ((size_t)c * H + h) * D * V;
-    int vc[VT];
 #pragma unroll
-    for (int j = 0; j < VT; j++) vc[j] = min(v0 + j * 16 + i16, V - 1);
-#pragma unroll 8
     for (int s = 0; s < DP / 4; s++) {
       const int d = 4 * s + k4;                    // queries are zero beyond D
-      const float* Sr = S + (size_t)min(d, D - 1) * V;
       const float a0 = sQ[(16 * I0 + i16) * LDQ + d] * sF[I0 * DP + d];
       const float a1 = sQ[(16 * I1 + i16) * LDQ + d] * sF[I1 * DP + d];
 #pragma unroll
       for (int j = 0; j < VT; j++) {
-        const float b = Sr[vc[j]];
-        acc[0][j] = mfma4(a0, b, acc[0][j]);
-        acc[1][j] = mfma4(a1, b, acc[1][j]);
+        acc[0][j] = mfma4(a0, S[s][j], acc[0][j]);
+        acc[1][j] = mfma4(a1, S[s][j], acc[1][j]);
       }
     }
 #pragma unroll

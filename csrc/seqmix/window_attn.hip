@@ -68,8 +68,8 @@ qk_norm_rope_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, i
   T* crow = pool ? pool + (size_t)cache_rows[r] * (nk + nv) : nullptr;
   T* qrow = q_out + (size_t)r * ldq;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-  // one wavefront per head: q heads, then k heads
-  for (int hh = wave; hh < heads; hh += nw) {
+  // one wavefront per head: q heads, then k heads (few rows: the heads of a row over several blocks)
+  for (int hh = blockIdx.y * nw + wave; hh < heads; hh += nw * gridDim.y) {
     const bool isq = hh < H;
     const int hd = isq ? hh : hh - H;
     const T* src = row + (isq ? 0 : nq) + hd * D;
@@ -98,7 +98,8 @@ qk_norm_rope_store_k(const T* __restrict__ proj, int ldp, int H, int G, int D, i
     for (int c = 2 * nrot + lane; c < D; c += 64) stf(dst, c, ldf(src, c) * rs * w[c]);
   }
   if (pool)
-    for (int i = threadIdx.x; i < nv; i += blockDim.x) crow[nk + i] = row[nq + nk + i];
+    for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < nv; i += blockDim.x * gridDim.y)
+      crow[nk + i] = row[nq + nk + i];
 }
 
 template <typename T>
@@ -112,15 +113,18 @@ __global__ void rope_rows_k(const T* __restrict__ src, int lds_, int heads, int 
   if (ro < 0) return;
   const T* s = src + (size_t)r * lds_;
   T* d = dst + ro * ldd;
-  for (int idx = threadIdx.x; idx < heads * nrot; idx += blockDim.x) {
-    int h = idx / nrot, i = idx % nrot;
-    float a = ldf(s, (size_t)h * src_hs + 2 * i), b = ldf(s, (size_t)h * src_hs + 2 * i + 1);
+  // a thread keeps one pair's angle for all the heads it walks
+  const int hstep = max((int)blockDim.x / nrot, 1);
+  for (int i = threadIdx.x % nrot, h0 = threadIdx.x / nrot; i < nrot && h0 < hstep; i += blockDim.x) {
     float sn, cs;
     sincosf(p * inv_freq[i], &sn, &cs);
     sn *= rm;
     cs *= rm;
-    stf(d, (size_t)(h * dst_hs + 2 * i), a * cs - b * sn);
-    stf(d, (size_t)(h * dst_hs + 2 * i + 1), b * cs + a * sn);
+    for (int h = h0; h < heads; h += hstep) {
+      float a = ldf(s, (size_t)h * src_hs + 2 * i), b = ldf(s, (size_t)h * src_hs + 2 * i + 1);
+      stf(d, (size_t)(h * dst_hs + 2 * i), a * cs - b * sn);
+      stf(d, (size_t)(h * dst_hs + 2 * i + 1), b * cs + a * sn);
+    }
   }
 }
 
@@ -372,7 +376,9 @@ int p2p_sm_qk_norm_rope_store(const void* proj, int ldp, int H, int G, int D, in
                               int f32, hipStream_t st) {
   if (R <= 0) return 0;
   if (H < 1 || G < 1 || D < 1 || V < 1 || nrot < 0 || 2 * nrot > D) return (int)hipErrorInvalidValue;
-  SM_DISPATCH_T(f32, hipLaunchKernelGGL(qk_norm_rope_store_k<T>, dim3(R), dim3(256), 0, st,
+  const int heads = pool ? H + G : H;
+  const dim3 grid(R, R <= 64 ? (heads + 3) / 4 : 1);
+  SM_DISPATCH_T(f32, hipLaunchKernelGGL(qk_norm_rope_store_k<T>, grid, dim3(256), 0, st,
                                          (const T*)proj, ldp, H, G, D, V, qw, kw, inv_freq, nrot,
                                          pos, cache_rows, (T*)pool, eps, (T*)q_out, ldq, per_head,
                                          half, rm));

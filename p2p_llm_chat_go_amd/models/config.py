@@ -176,7 +176,7 @@ def _hybrid_presets() -> dict:
          "eos_token_id": [2]}, name="tiny-rasepel"),
         "tiny-nosuzen": HybridConfig.from_dict(
         {"architecture": "Nosuzen", "width": 256, "vocab": 512, "norm": {"eps": 1e-6}, "streams": 4,
-         "embedding": {"scale": 1.0},
+         "embedding": {"scale": 2.0},
          "layers": [{"type": "attention", "mixer": da, "mlp": gmoe}, pg, dl,
                     {"type": "attention", "mixer": dict(da, kv_from=0), "mlp": gmoe}, dict(dl, mlp=None)],
          "eos_token_id": [2]}, name="tiny-nosuzen")}
