@@ -3,10 +3,11 @@
 //
 // conv_rope_norm_store_k: one projection buffer holds q (H heads x D) | k (G x D) | v (GV x V) of
 // every row (differential attention has two q / k heads, its maps, per value head; a layer that
-// reads another layer's keys and values has queries only, G = GV = 0).  Each channel goes through a causal convolution over the sequence's last K
-// projected values (those before the portion come from the slot's saved tail, or are zero before
+// reads another layer's keys and values has queries only, G = GV = 0).  Each channel goes through a
+// causal convolution over the sequence's last K projected values (those before the portion come from the slot's saved tail, or are zero before
 // position 0); nrot channel pairs (i, i + nrot) of every q / k head are turned by the angle
-// pos * inv_freq[i]; q and k heads are divided by their root mean square, sqrt(mean x^2 + eps) (`norm`);
+// pos * inv_freq[i] (cos and sin times rm); q and k heads are divided by their root mean square,
+// sqrt(mean x^2 + eps) (`norm`);
 // q also takes a factor per head (`temp`), which stands for a factor on that head's scores.  q
 // goes to its own buffer, k | v to the row of the paged pool that the token owns.  Convolution,
 // angles, rotation and norm are fp32.  One wavefront per (row, head).
@@ -23,7 +24,8 @@ using namespace sm;
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V, int norm,
+conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V,
+                       int norm, float rm,
                        const float* __restrict__ cw, int K, float* tail,
                        const int* __restrict__ ent, const int* __restrict__ row_ent,
                        const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
@@ -75,6 +77,8 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int GV
       const float a = s[j], b = s[j + nrot];
       float sn, cs;
       sincosf((float)p * inv_freq[j], &sn, &cs);
+      sn *= rm;
+      cs *= rm;
       const float x = a * cs - b * sn, y = b * cs + a * sn;
       s[j] = x;
       s[j + nrot] = y;
@@ -114,7 +118,8 @@ conv_rope_norm_store_k(const T* __restrict__ proj, int ldp, int H, int G, int GV
 #define RT 8
 template <typename T, int KT>
 __global__ void __launch_bounds__(256)
-conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V, int norm,
+conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int GV, int D, int V,
+                      int norm, float rm,
                       const float* __restrict__ cw, const float* __restrict__ tail,
                       const int* __restrict__ ent, const int* __restrict__ row_ent,
                       const float* __restrict__ inv_freq, int nrot, const float* __restrict__ temp,
@@ -128,8 +133,8 @@ conv_rope_norm_rows_k(const T* __restrict__ proj, int ldp, int H, int G, int GV,
   for (int idx = threadIdx.x; idx < nr * nrot; idx += 256) {
     float sn, cs;
     sincosf((float)pos[r0 + idx / nrot] * inv_freq[idx % nrot], &sn, &cs);
-    smem[2 * idx] = cs;
-    smem[2 * idx + 1] = sn;
+    smem[2 * idx] = cs * rm;
+    smem[2 * idx + 1] = sn * rm;
   }
   __syncthreads();
   const int C = (H + G) * D + GV * V, W = G * D + GV * V;
@@ -248,16 +253,16 @@ extern "C" {
 
 // rows: several rows per workgroup (3 or 4 taps, head sizes up to 256); the tails and blocks of
 // every portion, also of single tokens, are then left to other kernels
-int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int GV, int D, int V, int norm,
-                                const float* cw, int K, float* tail, const int* ent,
+int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int GV, int D, int V,
+                                int norm, float rm, const float* cw, int K, float* tail, const int* ent,
                                 const int* row_ent, const float* inv_freq, int nrot,
                                 const float* temp, float eps, const int* pos,
                                 const int* cache_rows, void* pool, void* q_out, int ldq, void* blk,
                                 int P, const int* bt, int max_pages, int page, int R, int rows,
                                 int f32, hipStream_t st) {
   if (R <= 0) return 0;
-  if (H < 1 || G < 0 || GV < 0 || (G + GV > 0 && !pool) || D < 1 || V < 1 || K < 1 || nrot < 0 || 2 * nrot > D || page < 1 ||
-      (blk && P < 1))
+  if (H < 1 || G < 0 || GV < 0 || (G + GV > 0 && !pool) || D < 1 || V < 1 || K < 1 || nrot < 0 ||
+      2 * nrot > D || page < 1 || (blk && P < 1))
     return (int)hipErrorInvalidValue;
   const int LDS = D > V ? D : V;
   if ((size_t)4 * LDS * 4 > 64 * 1024) return (int)hipErrorInvalidValue;
@@ -267,7 +272,8 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int GV,
     dim3 gr((R + RT - 1) / RT, (H + G + GV + 3) / 4);
 #define CRN(KT)                                                                                   \
   SM_DISPATCH_T(f32, hipLaunchKernelGGL((conv_rope_norm_rows_k<T, KT>), gr, dim3(256), shm, st,   \
-                                         (const T*)proj, ldp, H, G, GV, D, V, norm, cw, tail, ent, row_ent, \
+                                         (const T*)proj, ldp, H, G, GV, D, V, norm, rm, cw, tail, ent, \
+                                         row_ent,                                                 \
                                          inv_freq, nrot, temp, eps, pos, cache_rows, (T*)pool,    \
                                          (T*)q_out, ldq, R, LDS))
     if (K == 4) CRN(4);
@@ -277,7 +283,7 @@ int p2p_sm_conv_rope_norm_store(const void* proj, int ldp, int H, int G, int GV,
   }
   dim3 grid(R, (H + G + GV + 3) / 4);
   SM_DISPATCH_T(f32, hipLaunchKernelGGL(conv_rope_norm_store_k<T>, grid, dim3(256),
-                                         (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, GV, D, V, norm,
+                                         (size_t)4 * LDS * 4, st, (const T*)proj, ldp, H, G, GV, D, V, norm, rm,
                                          cw, K, tail, ent, row_ent, inv_freq, nrot, temp, eps, pos,
                                          cache_rows, (T*)pool, (T*)q_out, ldq, (T*)blk, P, bt,
                                          max_pages, page, LDS));

@@ -860,8 +860,7 @@ class DiffAttention(Mixer):
         lq1, lk1, lq2, lk2 = (get(k).double() for k in ("lq1", "lk1", "lq2", "lk2"))
         self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
         self.inv_freq = sm.rope_inv_freq(self.rot_base, self.rot_dims, dev, self.rot_scaling)
-        if sm.rope_magnitude(self.rot_scaling) != 1.0:
-            raise ValueError("diff_attention: the convolved input pass has no rotation magnitude")
+        self.rot_mag = sm.rope_magnitude(self.rot_scaling)
         self.wo = get("o").to(dev, dtype).contiguous()
 
     def cache_spec(self):
@@ -882,7 +881,7 @@ class DiffAttention(Mixer):
         q = torch.empty(b.R, H * 2 * D, device=proj.device, dtype=proj.dtype)
         sm.conv_rope_norm_store(proj, H, G, D, V, self.cw, cache.state[layer]["tail"], self.inv_freq, None,
                                 b.pos, b.cache_rows, pool if own else None, self.eps, q, b.ent, b.ent_host,
-                                b.row_ent, b.block_tables, PAGE, maps=2, norm=False)
+                                b.row_ent, b.block_tables, PAGE, maps=2, norm=False, rm=self.rot_mag)
         units = b.units(sm.window_rows_per_wave(H // G)) if sm.window_mfma_ok(q, pool, D, V) else None
         sm.window_attn(q, pool, b.block_tables, b.row_ent, b.pos, None, self.scale, self.win, out, PAGE,
                        H, G, D, V, units=units, max_keys=b.max_keys, out_scale=out_scale * (1.0 - self.diff),

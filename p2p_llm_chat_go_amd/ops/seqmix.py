@@ -1,15 +1,17 @@
 """Sequence-mixer ops: recurrent state layers (generalized delta rule, Mamba-2, the selective
-scan of the first Mamba, gated delta rule, HGRN2, lightning attention, the mLSTM's matrix memory),
+scan of the first Mamba, gated delta rule, HGRN2, lightning attention, gated linear attention, the
+mLSTM's matrix memory),
 latent attention (optionally with a rotated key part
 in the cached row and without a sink) and grouped-query attention with an optional sliding
 window and softmax sink (query/key norm over the row or per head, rotary positions on adjacent
 or half-split channel pairs and the cache write in one pass; or unrotated with a query
 temperature, capped scores, a logarithmic distance penalty and a gate per head; or behind short
 convolutions, with unit-RMS heads, pooled blocks of the tokens before the window and a gate per
-channel), a group-limited expert router (sigmoid or softmax scores, optional score correction and bias,
-softmax over the chosen logits) with grouped expert products and identity experts, learned
+channel; or differential, two maps per head on the same values, and windows that keep the first
+tokens), a group-limited expert router (sigmoid or softmax scores, optional score correction and bias,
+softmax over the chosen logits, rescaled weights) with grouped expert products and identity experts, learned
 positions, and the norms, residual passes (one with two normed outputs and the routed experts'
-weighted sum) and pointwise steps around them.
+weighted sum, one over parallel residual streams with a dynamic tanh) and pointwise steps around them.
 
 GPU tensors always run the gfx950 kernels of ``csrc/seqmix`` (``libp2p_seqmix.so``, built on
 first use when missing); CPU tensors run the PyTorch rendering of the same math, which is
@@ -70,7 +72,8 @@ _SIGS = {
                               c_int, c_int, c_int, c_int, c_void_p],
     "p2p_sm_lightning_chunked": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
                                  c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
-    "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
+    "p2p_sm_conv_rope_norm_store": [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                                    c_void_p, c_int,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_float,
                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int,
                                     c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
@@ -1307,13 +1310,13 @@ def blocks_per_page(page: int, every: int) -> int:
 def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_freq, temp, pos,
                          cache_rows, pool, eps: float, q_out, ent, ent_host, row_ent,
                          block_tables, page: int, blk=None, every: int = 0, maps: int = 1,
-                         norm: bool = True):
+                         norm: bool = True, rm: float = 1.0):
     """Prepares attention inputs from one projection buffer proj = [q (H*D) | k (G*D) | v (G*V) | ..]:
     every channel goes through a causal convolution over time (cw fp32 [C, K], column K-1 the newest
     input, no bias; tail fp32 [slots, K-1, C] the projections before each slot's next token, moved
     forward here), the pairs (i, i + nrot), i < nrot = len(inv_freq), of every q and k head are turned
-    by pos * inv_freq[i], q and k heads are divided by sqrt(mean(x^2) + eps), and q head h is multiplied
-    by temp[h] (fp32 [H] or None).  q goes to q_out [R, H*D], k | v to the rows ``cache_rows`` of the
+    by pos * inv_freq[i] (cos and sin times rm), q and k heads are divided by sqrt(mean(x^2) + eps), and
+    q head h is multiplied by temp[h] (fp32 [H] or None).  q goes to q_out [R, H*D], k | v to the rows ``cache_rows`` of the
     paged pool.  All of it fp32.
     blk: a pool of blocks of ``every`` tokens ([pages * blocks_per_page, G*(D+V)]); the blocks that
     this step's tokens complete get the mean of their tokens' rows of ``pool``.
@@ -1335,7 +1338,7 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
             y[row0:row0 + n] = sum(pad[kk:kk + n] * cw[:, kk] for kk in range(K))
         conv_tail_roll(proj, 0, tail, ent, ent_host, C)
         ang = pos[:R].float()[:, None] * inv_freq[None, :]
-        c, sn = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+        c, sn = torch.cos(ang)[:, None, :] * rm, torch.sin(ang)[:, None, :] * rm
 
         def prep(t, heads):
             t = t.reshape(R, heads, D).clone()
@@ -1385,7 +1388,7 @@ def conv_rope_norm_store(proj, H: int, G: int, D: int, V: int, cw, tail, inv_fre
     # single tokens move their tails and form their blocks in the first kernel
     rows = R >= 64 and K in (3, 4) and max(D, V) <= 256 and any(e[1] > 1 for e in ent_host)
     _chk(lib().p2p_sm_conv_rope_norm_store(
-        proj.data_ptr(), proj.stride(0), HQ, GK, GV, D, V, 1 if norm else 0, cw.data_ptr(), K, tail.data_ptr(),
+        proj.data_ptr(), proj.stride(0), HQ, GK, GV, D, V, 1 if norm else 0, rm, cw.data_ptr(), K, tail.data_ptr(),
         ent.data_ptr(), row_ent.data_ptr(), inv_freq.data_ptr(), nrot, _lib.ptr(temp), eps,
         pos.data_ptr(), cache_rows.data_ptr(), _lib.ptr(pool), q_out.data_ptr(), q_out.stride(0),
         _lib.ptr(blk), every, block_tables.data_ptr(), block_tables.shape[1], page, R,

@@ -111,7 +111,7 @@ def test_two_map_input_pass(dt, H, G, D, V, K, dims, step):
             pool, tail, q = pool0.clone().to(dev), tail0.clone().to(dev), torch.empty(R, 2 * H * D, dtype=dt, device=dev)
             sm.conv_rope_norm_store(proj.to(dev), H, G, D, V, cw.to(dev), tail, inv.to(dev), None, pos.to(dev),
                                     rows.to(dev), pool if own else None, 1e-3, q, entt.to(dev), ent, row_ent.to(dev),
-                                    pages.to(dev), PAGE, maps=2, norm=False)
+                                    pages.to(dev), PAGE, maps=2, norm=False, rm=1.2)
             res.append((q.cpu(), pool.cpu(), tail.cpu()))
         torch.testing.assert_close(res[1][0].float(), res[0][0].float(), **_tol(dt))
         torch.testing.assert_close(res[1][1].float(), res[0][1].float(), **_tol(dt))
